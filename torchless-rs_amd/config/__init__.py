@@ -6,7 +6,9 @@ from .sozetar import SozetarConfig
 from .fanitar import FanitarConfig
 from .nepisun import NepisunConfig
 from .giforax import GiforaxConfig
+from .zudalorn import ZudalornConfig
 
-__all__ = ["ArchitectureEntry", "ConfigError", "ModelConfig", "MistralConfig", "SozetarConfig", "FanitarConfig", "NepisunConfig", "GiforaxConfig", "architecture_name",
+__all__ = ["ArchitectureEntry", "ConfigError", "ModelConfig", "MistralConfig", "SozetarConfig", "FanitarConfig", "NepisunConfig", "GiforaxConfig",
+           "ZudalornConfig", "architecture_name",
            "config_from_dict", "get_architecture", "load_config", "register_architecture",
            "registered_architectures", "unregister_architecture"]

@@ -84,6 +84,7 @@ struct Rotation {
   const float* inv_freq;   // [rotary_dim / 2]
   int rotary_dim;
   int interleaved;         // pairs (2i, 2i+1); else (i, i + rotary_dim/2)
+  float magnitude = 1.f;   // a factor on both cosine and sine (the kernels that take one say so)
 };
 // The two channels of pair i of a head, i < d/2.  Pairs from rotary_dim/2 on are not rotated;
 // they are numbered so that the d/2 pairs cover every channel once.

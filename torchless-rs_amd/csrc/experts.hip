@@ -1,11 +1,13 @@
 // A routed mixture of small feed-forward layers ("experts").
 //
 // Router, per row, in float: z = W_r h, s = softmax(z) over all E experts (or, `logistic`, every
-// expert's own 1 / (1 + exp(-z))).  The experts form
-// `groups` equal groups of neighbours; a group's score is its largest s, and only experts of the
-// `keep` best groups can be chosen (groups == 0: every expert can).  Of those the `top` with the
-// largest s are chosen; their weights are their s, not renormalised.  Of equal scores the one
-// with the smaller index goes first.
+// expert's own 1 / (1 + exp(-z))).  The choice goes by c = s, or c = s + correction[e] (which may be
+// negative).  The experts form `groups` equal groups of neighbours; a group's score is its largest
+// c, or the sum of its two largest (`two_largest`), and only experts of the `keep` best groups can be
+// chosen (groups == 0: every expert can).  Of those the `top` with the largest c are chosen; their
+// weights are their s, as they are or divided by (their sum + normalise_eps) (`normalise`).  Of equal
+// scores the one with the smaller index goes first.  A shared expert may have a weight of its own, the
+// logistic function of one more row of the router's matrix (`shared_weight`).
 //
 // `route` leaves the weights as a row of E floats, zero for an expert that was not chosen.
 // The experts run as ONE wide feed-forward: the rows of all up projections stacked (the shared
@@ -20,18 +22,28 @@ constexpr int RT_MAX_E = 1024;
 
 // NT threads a row: a quarter of a thousand, or 1024 for steps of few rows, where a row's dots are what the step waits
 // for (16 waves take 16 experts at a time instead of 4).  A dot is one wave's either way: the same bits.
+struct RouteTerms {
+  const float* correction;   // [E] or null
+  int two_largest;
+  int normalise;
+  float normalise_eps;
+  float* shared_weight;      // [n] or null; with it the router's matrix has a row E
+};
+
 template <typename T, int NT>
 __global__ void __launch_bounds__(NT)
 route_kernel(const T* __restrict__ h, int W, const float* __restrict__ wr, int E, int groups, int keep, int top,
-             int logistic, float* __restrict__ weights, int* __restrict__ chosen, bool vec) {
-  __shared__ float s_s[RT_MAX_E];
+             int logistic, RouteTerms k, float* __restrict__ weights, int* __restrict__ chosen, bool vec) {
+  __shared__ float s_s[RT_MAX_E + 1];
+  __shared__ float c_s[RT_MAX_E];          // what the choice goes by
   __shared__ float g_s[RT_MAX_E];
   __shared__ unsigned char ok_s[RT_MAX_E];
   __shared__ float sh[NT / WAVE];
   const int n = blockIdx.x;
   const int t = threadIdx.x, lane = t % WAVE, wave = t / WAVE;
   const T* row = h + (size_t)n * W;
-  for (int e = wave; e < E; e += NT / WAVE) {
+  const int rows = E + (k.shared_weight ? 1 : 0);
+  for (int e = wave; e < rows; e += NT / WAVE) {
     const float* w = wr + (size_t)e * W;
     float d0 = 0.f, d1 = 0.f, d2 = 0.f, d3 = 0.f;      // four chains: the loads of one do not wait for another's sum
     int c = 0;
@@ -59,6 +71,7 @@ route_kernel(const T* __restrict__ h, int W, const float* __restrict__ wr, int E
     if (lane == 0) s_s[e] = dot;
   }
   __syncthreads();
+  if (k.shared_weight && t == 0) k.shared_weight[n] = 1.0f / (1.0f + expf(-s_s[E]));
   if (logistic) {                                      // every expert's score by itself
     for (int e = t; e < E; e += NT) s_s[e] = 1.0f / (1.0f + expf(-s_s[e]));
   } else {
@@ -72,12 +85,18 @@ route_kernel(const T* __restrict__ h, int W, const float* __restrict__ wr, int E
     for (int e = t; e < E; e += NT) s_s[e] = expf(s_s[e] - m) / sum;
   }
   __syncthreads();
+  for (int e = t; e < E; e += NT) c_s[e] = s_s[e] + (k.correction ? k.correction[e] : 0.f);
+  __syncthreads();
   if (groups > 0) {
     const int per = E / groups;
     for (int g = t; g < groups; g += NT) {
-      float best = s_s[g * per];
-      for (int i = 1; i < per; ++i) best = fmaxf(best, s_s[g * per + i]);
-      g_s[g] = best;
+      float best = c_s[g * per], second = -INFINITY;
+      for (int i = 1; i < per; ++i) {
+        const float c = c_s[g * per + i];
+        second = fmaxf(second, fminf(best, c));
+        best = fmaxf(best, c);
+      }
+      g_s[g] = k.two_largest && per > 1 ? best + second : best;
     }
     __syncthreads();
     for (int g = t; g < groups; g += NT) {
@@ -90,32 +109,53 @@ route_kernel(const T* __restrict__ h, int W, const float* __restrict__ wr, int E
     for (int e = t; e < E; e += NT) ok_s[e] = 1;
   }
   __syncthreads();
+  float mine_sum = 0.f;
   for (int e = t; e < E; e += NT) {
     float wgt = 0.f;
     if (ok_s[e]) {
       int ahead = 0;
-      const float mine = s_s[e];
-      for (int o = 0; o < E; ++o) ahead += (ok_s[o] && (s_s[o] > mine || (s_s[o] == mine && o < e))) ? 1 : 0;
+      const float mine = c_s[e];
+      for (int o = 0; o < E; ++o) ahead += (ok_s[o] && (c_s[o] > mine || (c_s[o] == mine && o < e))) ? 1 : 0;
       if (ahead < top) {
-        wgt = mine;
+        wgt = s_s[e];
         if (chosen) chosen[(size_t)n * top + ahead] = e;
       }
     }
-    weights[(size_t)n * E + e] = wgt;
+    if (k.normalise) {
+      g_s[e] = wgt;                        // (the groups' scores have been read)
+      mine_sum += wgt;
+    } else {
+      weights[(size_t)n * E + e] = wgt;
+    }
+  }
+  if (k.normalise) {
+    const float sum = block_sum<NT>(mine_sum, sh) + k.normalise_eps;
+    for (int e = t; e < E; e += NT) weights[(size_t)n * E + e] = g_s[e] / sum;      // (a thread's own entries)
   }
 }
 
-// out[n, j] = act(u[n, j]) * (j < E * ff ? weights[n, j / ff] : 1), act = the square of max(., 0)
-// (code 0) or max(., 0) (code 1).
+// act = the square of max(., 0) (code 0), max(., 0) (code 1), or xIELU (code 2) with two numbers a and b:
+// a z^2 + z/2 where z > 0, b (exp(z) - 1 - z) + z/2 elsewhere
+struct UnaryAct {
+  int code;
+  float a, b;
+};
+__device__ __forceinline__ float unary_act(float z, const UnaryAct& k) {
+  if (k.code == 2) return z > 0.f ? fmaf(k.a * z, z, 0.5f * z) : fmaf(k.b, expm1f(z) - z, 0.5f * z);
+  const float r = fmaxf(z, 0.f);
+  return k.code == 0 ? r * r : r;
+}
+
+// out[n, j] = act(u[n, j]) * (j < E * ff ? weights[n, j / ff] : shared_w ? shared_w[n] : 1)
 template <typename T>
 __global__ void __launch_bounds__(256)
-expert_act_kernel(const float* __restrict__ u, const float* __restrict__ weights, int E, int ff, int total, int act,
-                  T* __restrict__ out) {
+expert_act_kernel(const float* __restrict__ u, const float* __restrict__ weights, const float* __restrict__ shared_w, int E,
+                  int ff, int total, UnaryAct act, T* __restrict__ out) {
   const int n = blockIdx.x;
   for (int j = blockIdx.y * 256 + threadIdx.x; j < total; j += gridDim.y * 256) {
-    float a = fmaxf(u[(size_t)n * total + j], 0.f);
-    if (act == 0) a *= a;
+    float a = unary_act(u[(size_t)n * total + j], act);
     if (j < E * ff) a *= weights[(size_t)n * E + j / ff];
+    else if (shared_w) a *= shared_w[n];
     out[(size_t)n * total + j] = from_f32<T>(a);
   }
 }
@@ -161,8 +201,8 @@ constexpr int ER_ROWS = 16;      // outputs of a workgroup: four a wave
 template <typename T>
 __global__ void __launch_bounds__(256)
 expert_rows_up_kernel(const T* __restrict__ y, int H, const T* __restrict__ up, const int* __restrict__ chosen,
-                      const float* __restrict__ weights, int E, int top, int ff, int shared, int act, bool vec,
-                      T* __restrict__ hs) {
+                      const float* __restrict__ weights, const float* __restrict__ shared_w, int E, int top, int ff, int shared,
+                      UnaryAct act, bool vec, T* __restrict__ hs) {
   const int slots = top + (shared ? 1 : 0);
   const int n = blockIdx.x / slots, k = blockIdx.x % slots;
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
@@ -176,6 +216,7 @@ expert_rows_up_kernel(const T* __restrict__ y, int H, const T* __restrict__ up, 
   } else {
     base = E * ff;
     count = shared;
+    if (shared_w) scale = shared_w[n];
   }
   const T* row = y + (size_t)n * H;
   T* out = hs + (size_t)n * (top * ff + shared) + (size_t)k * ff;
@@ -183,8 +224,7 @@ expert_rows_up_kernel(const T* __restrict__ y, int H, const T* __restrict__ up, 
   for (int r = 0; r < ER_ROWS / 4; ++r) {
     const int j = blockIdx.y * ER_ROWS + wave * (ER_ROWS / 4) + r;
     if (j >= count) break;
-    float a = fmaxf(wave_dot(up + (size_t)(base + j) * H, row, H, vec, lane), 0.f);
-    if (act == 0) a *= a;
+    const float a = unary_act(wave_dot(up + (size_t)(base + j) * H, row, H, vec, lane), act);
     if (lane == 0) out[j] = from_f32<T>(a * scale);
   }
 }
@@ -242,8 +282,8 @@ __device__ __forceinline__ float gated_value(float g, float u, float s, float li
 // lays it; weights [n, E] (E == 0: none; a column of weight 1 for the shared part)
 template <typename T>
 __global__ void __launch_bounds__(256)
-expert_gated_act_kernel(const float* __restrict__ gu, const float* __restrict__ weights, int E, int ff, int shared,
-                        GateTerms k, T* __restrict__ out) {
+expert_gated_act_kernel(const float* __restrict__ gu, const float* __restrict__ weights, const float* __restrict__ shared_w,
+                        int E, int ff, int shared, GateTerms k, T* __restrict__ out) {
   const int n = blockIdx.x;
   const int total = E * ff + shared;
   const float* row = gu + (size_t)n * 2 * total;
@@ -255,6 +295,7 @@ expert_gated_act_kernel(const float* __restrict__ gu, const float* __restrict__ 
     } else {
       const int c = j - E * ff;
       a = gated_value(row[2 * E * ff + c], row[2 * E * ff + shared + c], 1.f, k.limit_shared, k);
+      if (shared_w) a *= shared_w[n];
     }
     out[(size_t)n * total + j] = from_f32<T>(a);
   }
@@ -265,13 +306,13 @@ expert_gated_act_kernel(const float* __restrict__ gu, const float* __restrict__ 
 template <typename T>
 __global__ void __launch_bounds__(256)
 expert_rows_gated_up_kernel(const T* __restrict__ y, int H, const T* __restrict__ up, const int* __restrict__ chosen,
-                            const float* __restrict__ weights, int E, int top, int ff, int shared, GateTerms kt, bool vec,
-                            T* __restrict__ hs) {
+                            const float* __restrict__ weights, const float* __restrict__ shared_w, int E, int top, int ff,
+                            int shared, GateTerms kt, bool vec, T* __restrict__ hs) {
   const int slots = top + (shared ? 1 : 0);
   const int n = blockIdx.x / slots, k = blockIdx.x % slots;
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
   int base, count;
-  float scale = 1.f, limit = kt.limit_shared;
+  float scale = 1.f, limit = kt.limit_shared, after = 1.f;     // after: the shared expert's own weight, on its output
   if (k < top) {
     const int e = chosen[(size_t)n * top + k];
     base = 2 * e * ff;
@@ -281,6 +322,7 @@ expert_rows_gated_up_kernel(const T* __restrict__ y, int H, const T* __restrict_
   } else {
     base = 2 * E * ff;
     count = shared;
+    if (shared_w) after = shared_w[n];
   }
   const T* row = y + (size_t)n * H;
   T* out = hs + (size_t)n * (top * ff + shared) + (size_t)k * ff;
@@ -290,7 +332,7 @@ expert_rows_gated_up_kernel(const T* __restrict__ y, int H, const T* __restrict_
     if (j >= count) break;
     const float g = wave_dot(up + (size_t)(base + j) * H, row, H, vec, lane);
     const float u = wave_dot(up + (size_t)(base + count + j) * H, row, H, vec, lane);
-    if (lane == 0) out[j] = from_f32<T>(gated_value(g, u, scale, limit, kt));
+    if (lane == 0) out[j] = from_f32<T>(gated_value(g, u, scale, limit, kt) * after);
   }
 }
 
@@ -301,7 +343,8 @@ using namespace tl;
 extern "C" {
 
 int tl_route(const void* h, int dt, int n, int W, const float* wr, int E, int groups, int keep, int top, int logistic,
-             float* weights, int* chosen, hipStream_t st) {
+             const float* correction, int two_largest, int normalise, float normalise_eps, float* shared_weight, float* weights,
+             int* chosen, hipStream_t st) {
   TL_REQUIRE(n >= 0 && W > 0 && E > 0 && E <= RT_MAX_E && top > 0 && top <= E, "route: bad sizes n=%d W=%d E=%d top=%d (experts up to %d)",
              n, W, E, top, RT_MAX_E);
   TL_REQUIRE(groups >= 0 && (groups == 0 || (E % groups == 0 && keep > 0 && keep <= groups && keep * (E / groups) >= top)),
@@ -310,30 +353,32 @@ int tl_route(const void* h, int dt, int n, int W, const float* wr, int E, int gr
   if (n == 0) return 0;
   const bool vec = W % 4 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)wr % 16 == 0;
   TL_REQUIRE(dt == DT_F32 || dt == DT_BF16, "route: unknown dtype code %d", dt);
+  const RouteTerms k{correction, two_largest, normalise, normalise_eps, shared_weight};
   const bool few = n <= 64 && E > 4;             // fewer rows than compute units: more waves a row
   if (dt == DT_F32 && few)
-    route_kernel<float, 1024><<<n, 1024, 0, st>>>((const float*)h, W, wr, E, groups, keep, top, logistic, weights, chosen, vec);
+    route_kernel<float, 1024><<<n, 1024, 0, st>>>((const float*)h, W, wr, E, groups, keep, top, logistic, k, weights, chosen, vec);
   else if (dt == DT_F32)
-    route_kernel<float, 256><<<n, 256, 0, st>>>((const float*)h, W, wr, E, groups, keep, top, logistic, weights, chosen, vec);
+    route_kernel<float, 256><<<n, 256, 0, st>>>((const float*)h, W, wr, E, groups, keep, top, logistic, k, weights, chosen, vec);
   else if (few)
-    route_kernel<bf16, 1024><<<n, 1024, 0, st>>>((const bf16*)h, W, wr, E, groups, keep, top, logistic, weights, chosen, vec);
+    route_kernel<bf16, 1024><<<n, 1024, 0, st>>>((const bf16*)h, W, wr, E, groups, keep, top, logistic, k, weights, chosen, vec);
   else
-    route_kernel<bf16, 256><<<n, 256, 0, st>>>((const bf16*)h, W, wr, E, groups, keep, top, logistic, weights, chosen, vec);
+    route_kernel<bf16, 256><<<n, 256, 0, st>>>((const bf16*)h, W, wr, E, groups, keep, top, logistic, k, weights, chosen, vec);
   TL_LAUNCH_CHECK("route");
   return 0;
 }
 
-int tl_expert_act(const float* u, const float* weights, int n, int E, int ff, int total, int act, void* out, int dt,
-                  hipStream_t st) {
-  TL_REQUIRE(n >= 0 && E >= 0 && ff > 0 && total >= E * ff && (act == 0 || act == 1), "expert_act: bad sizes E=%d ff=%d total=%d act=%d",
-             E, ff, total, act);
+int tl_expert_act(const float* u, const float* weights, const float* shared_w, int n, int E, int ff, int total, int act_code,
+                  float act_a, float act_b, void* out, int dt, hipStream_t st) {
+  const UnaryAct act{act_code, act_a, act_b};
+  TL_REQUIRE(n >= 0 && E >= 0 && ff > 0 && total >= E * ff && act_code >= 0 && act_code <= 2, "expert_act: bad sizes E=%d ff=%d total=%d act=%d",
+             E, ff, total, act_code);
   TL_REQUIRE(u && out && (E == 0 || weights), "expert_act: a buffer is missing");
   if (n == 0) return 0;
   const dim3 grid(n, min((total + 255) / 256, 64));
   if (dt == DT_F32)
-    expert_act_kernel<float><<<grid, 256, 0, st>>>(u, weights, E, ff, total, act, (float*)out);
+    expert_act_kernel<float><<<grid, 256, 0, st>>>(u, weights, shared_w, E, ff, total, act, (float*)out);
   else if (dt == DT_BF16)
-    expert_act_kernel<bf16><<<grid, 256, 0, st>>>(u, weights, E, ff, total, act, (bf16*)out);
+    expert_act_kernel<bf16><<<grid, 256, 0, st>>>(u, weights, shared_w, E, ff, total, act, (bf16*)out);
   else
     TL_REQUIRE(false, "expert_act: unknown dtype code %d", dt);
   TL_LAUNCH_CHECK("expert_act");
@@ -341,10 +386,11 @@ int tl_expert_act(const float* u, const float* weights, int n, int E, int ff, in
 }
 
 // y [n, H], up [E * ff + shared, H], chosen int [n, top], weights [n, E] -> hs [n, top * ff + shared], all of dtype dt
-int tl_expert_rows_up(const void* y, int H, const void* up, const int* chosen, const float* weights, int n, int E, int top, int ff,
-                      int shared, int act, void* hs, int dt, hipStream_t st) {
-  TL_REQUIRE(n >= 0 && H > 0 && E > 0 && top > 0 && top <= E && ff > 0 && shared >= 0 && (act == 0 || act == 1),
-             "expert_rows_up: bad sizes H=%d E=%d top=%d ff=%d shared=%d act=%d", H, E, top, ff, shared, act);
+int tl_expert_rows_up(const void* y, int H, const void* up, const int* chosen, const float* weights, const float* shared_w, int n, int E,
+                      int top, int ff, int shared, int act_code, float act_a, float act_b, void* hs, int dt, hipStream_t st) {
+  const UnaryAct act{act_code, act_a, act_b};
+  TL_REQUIRE(n >= 0 && H > 0 && E > 0 && top > 0 && top <= E && ff > 0 && shared >= 0 && act_code >= 0 && act_code <= 2,
+             "expert_rows_up: bad sizes H=%d E=%d top=%d ff=%d shared=%d act=%d", H, E, top, ff, shared, act_code);
   TL_REQUIRE(y && up && chosen && weights && hs, "expert_rows_up: a buffer is missing");
   TL_REQUIRE(dt == DT_F32 || dt == DT_BF16, "expert_rows_up: unknown dtype code %d", dt);
   if (n == 0) return 0;
@@ -354,10 +400,10 @@ int tl_expert_rows_up(const void* y, int H, const void* up, const int* chosen, c
   const int per = dt == DT_BF16 ? 8 : 4;
   const bool vec = H % per == 0 && (uintptr_t)y % 16 == 0 && (uintptr_t)up % 16 == 0;
   if (dt == DT_F32)
-    expert_rows_up_kernel<float><<<grid, 256, 0, st>>>((const float*)y, H, (const float*)up, chosen, weights, E, top, ff, shared, act, vec,
+    expert_rows_up_kernel<float><<<grid, 256, 0, st>>>((const float*)y, H, (const float*)up, chosen, weights, shared_w, E, top, ff, shared, act, vec,
                                                        (float*)hs);
   else
-    expert_rows_up_kernel<bf16><<<grid, 256, 0, st>>>((const bf16*)y, H, (const bf16*)up, chosen, weights, E, top, ff, shared, act, vec,
+    expert_rows_up_kernel<bf16><<<grid, 256, 0, st>>>((const bf16*)y, H, (const bf16*)up, chosen, weights, shared_w, E, top, ff, shared, act, vec,
                                                       (bf16*)hs);
   TL_LAUNCH_CHECK("expert_rows_up");
   return 0;
@@ -383,7 +429,7 @@ int tl_expert_rows_down(const void* hs, const void* down, const int* chosen, int
 }
 
 // gu float [n, 2 (E * ff + shared)], weights float [n, E] (E == 0: none) -> out [n, E * ff + shared] of dtype dt
-int tl_expert_gated_act(const float* gu, const float* weights, int n, int E, int ff, int shared, float limit, float limit_shared,
+int tl_expert_gated_act(const float* gu, const float* weights, const float* shared_w, int n, int E, int ff, int shared, float limit, float limit_shared,
                         float alpha, float shift, int on_input, void* out, int dt, hipStream_t st) {
   TL_REQUIRE(n >= 0 && E >= 0 && ff >= 0 && shared >= 0 && E * ff + shared > 0, "expert_gated_act: bad sizes E=%d ff=%d shared=%d", E, ff, shared);
   TL_REQUIRE(gu && out && (E == 0 || weights), "expert_gated_act: a buffer is missing");
@@ -392,15 +438,15 @@ int tl_expert_gated_act(const float* gu, const float* weights, int n, int E, int
   const int total = E * ff + shared;
   const dim3 grid(n, min((total + 255) / 256, 64));
   const GateTerms k{limit, limit_shared, alpha, shift, on_input};
-  if (dt == DT_F32) expert_gated_act_kernel<float><<<grid, 256, 0, st>>>(gu, weights, E, ff, shared, k, (float*)out);
-  else expert_gated_act_kernel<bf16><<<grid, 256, 0, st>>>(gu, weights, E, ff, shared, k, (bf16*)out);
+  if (dt == DT_F32) expert_gated_act_kernel<float><<<grid, 256, 0, st>>>(gu, weights, shared_w, E, ff, shared, k, (float*)out);
+  else expert_gated_act_kernel<bf16><<<grid, 256, 0, st>>>(gu, weights, shared_w, E, ff, shared, k, (bf16*)out);
   TL_LAUNCH_CHECK("expert_gated_act");
   return 0;
 }
 
 // y [n, H], up [2 (E * ff + shared), H], chosen int [n, top], weights [n, E] -> hs [n, top * ff + shared], all of dtype dt
-int tl_expert_rows_gated_up(const void* y, int H, const void* up, const int* chosen, const float* weights, int n, int E, int top,
-                            int ff, int shared, float limit, float limit_shared, float alpha, float shift, int on_input, void* hs,
+int tl_expert_rows_gated_up(const void* y, int H, const void* up, const int* chosen, const float* weights, const float* shared_w, int n,
+                            int E, int top, int ff, int shared, float limit, float limit_shared, float alpha, float shift, int on_input, void* hs,
                             int dt, hipStream_t st) {
   TL_REQUIRE(n >= 0 && H > 0 && E > 0 && top > 0 && top <= E && ff > 0 && shared >= 0,
              "expert_rows_gated_up: bad sizes H=%d E=%d top=%d ff=%d shared=%d", H, E, top, ff, shared);
@@ -414,10 +460,10 @@ int tl_expert_rows_gated_up(const void* y, int H, const void* up, const int* cho
   const bool vec = H % per == 0 && (uintptr_t)y % 16 == 0 && (uintptr_t)up % 16 == 0;
   const GateTerms k{limit, limit_shared, alpha, shift, on_input};
   if (dt == DT_F32)
-    expert_rows_gated_up_kernel<float><<<grid, 256, 0, st>>>((const float*)y, H, (const float*)up, chosen, weights, E, top, ff, shared, k,
+    expert_rows_gated_up_kernel<float><<<grid, 256, 0, st>>>((const float*)y, H, (const float*)up, chosen, weights, shared_w, E, top, ff, shared, k,
                                                              vec, (float*)hs);
   else
-    expert_rows_gated_up_kernel<bf16><<<grid, 256, 0, st>>>((const bf16*)y, H, (const bf16*)up, chosen, weights, E, top, ff, shared, k,
+    expert_rows_gated_up_kernel<bf16><<<grid, 256, 0, st>>>((const bf16*)y, H, (const bf16*)up, chosen, weights, shared_w, E, top, ff, shared, k,
                                                             vec, (bf16*)hs);
   TL_LAUNCH_CHECK("expert_rows_gated_up");
   return 0;

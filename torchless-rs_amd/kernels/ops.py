@@ -136,20 +136,27 @@ class Rotation:
     """How q and k are rotated by position: the first `rotary_dim` channels of a head in pairs,
     pair i by the angle pos * inv_freq[i] (float32 [rotary_dim / 2] on the device); pairs are
     (i, i + rotary_dim/2), or (2i, 2i+1) when `interleaved`; the channels behind them pass
-    through.  rotary_dim 0 (inv_freq None): nothing is rotated."""
+    through.  rotary_dim 0 (inv_freq None): nothing is rotated.  `magnitude`: a factor on both cosine
+    and sine, hence on the rotated channels alone (served by `retention_scan`, `retention_prepare` and
+    `latent_prepare`; the other kernels refuse one that is not 1)."""
 
-    def __init__(self, inv_freq: Optional[torch.Tensor], rotary_dim: int, interleaved: bool = False):
+    def __init__(self, inv_freq: Optional[torch.Tensor], rotary_dim: int, interleaved: bool = False,
+                 magnitude: float = 1.0):
         self.inv_freq, self.rotary_dim, self.interleaved = inv_freq, int(rotary_dim), bool(interleaved)
+        self.magnitude = float(magnitude)
 
 
 NO_ROTATION = Rotation(None, 0)
 
 
-def _rotation(rot, d: int, what: str) -> Rotation:
+def _rotation(rot, d: int, what: str, magnitude: bool = False) -> Rotation:
     """A `Rotation` checked against the head size `d`.  A bare tensor of d/2 frequencies stands
-    for the rotation of the whole head in halves; None for no rotation."""
+    for the rotation of the whole head in halves; None for no rotation.  `magnitude`: does the
+    kernel take a factor on cosines and sines?"""
     if rot is None:
         return NO_ROTATION
+    if not magnitude and isinstance(rot, Rotation) and rot.magnitude != 1.0:
+        raise KernelError(f"{what}: a factor of {rot.magnitude} on the rotated channels is not served")
     if isinstance(rot, torch.Tensor):
         rot = Rotation(rot, d)
     if rot.rotary_dim % 2 or not (0 <= rot.rotary_dim <= d):
@@ -911,31 +918,58 @@ def ssm_gate_norm(y: torch.Tensor, proj: torch.Tensor, parts: int, w: torch.Tens
 
 
 # ---- routed experts ----------------------------------------------------------------------------------
-EXPERT_ACTIVATIONS = {"relu2": 0, "relu": 1}
+EXPERT_ACTIVATIONS = {"relu2": 0, "relu": 1, "xielu": 2}
+UNARY_CONSTANTS = {"xielu": ("a", "b")}      # activations with numbers of their own, in the kernels' order
+
+
+def _unary_args(activation: str, constants):
+    """Code and constants of an activation of one argument, as the kernels take them."""
+    if activation not in EXPERT_ACTIVATIONS:
+        raise KernelError(f"no function {activation!r}; there are {sorted(EXPERT_ACTIVATIONS)}")
+    need = UNARY_CONSTANTS.get(activation, ())
+    if set(constants or {}) != set(need):
+        raise KernelError(f"{activation!r} takes the constants {sorted(need)}, got {sorted(constants or {})}")
+    k = [float(constants[n]) for n in need] + [0.0] * (2 - len(need))
+    return EXPERT_ACTIVATIONS[activation], ctypes.c_float(k[0]), ctypes.c_float(k[1])
+
+
+def _shared_weight(w: Optional[torch.Tensor], n: int, what: str):
+    if w is not None:
+        _req(w, what + ".shared_weight", torch.float32, (n,))
+    return _p(w)
 
 
 def route(h: torch.Tensor, router: torch.Tensor, groups: int, keep: int, top: int, weights: torch.Tensor,
-          chosen: Optional[torch.Tensor] = None, logistic: bool = False) -> None:
+          chosen: Optional[torch.Tensor] = None, logistic: bool = False, correction: Optional[torch.Tensor] = None,
+          two_largest: bool = False, normalise_eps: Optional[float] = None,
+          shared_weight: Optional[torch.Tensor] = None) -> None:
     """The router of a mixture of experts, in float32: s = softmax(router h) over the E experts (`logistic`:
-    every expert's own 1 / (1 + exp(-router h)) instead); of the `keep`
-    groups (of `groups` equal groups of neighbours; 0: no groups) whose best s is largest, the `top` experts
-    with the largest s; `weights` float32 [n, E] receives s for those and 0 for the others, `chosen` (int32
-    [n, top], or None) their indices, the best first."""
+    every expert's own 1 / (1 + exp(-router h)) instead).  The choice goes by c = s (+ `correction`, float32 [E]):
+    of the `keep` groups (of `groups` equal groups of neighbours; 0: no groups) whose best c is largest
+    (`two_largest`: the sum of whose two best is), the `top` experts with the largest c; `weights` float32
+    [n, E] receives s for those (with `normalise_eps`: divided by (their sum + normalise_eps)) and 0 for the
+    others, `chosen` (int32 [n, top], or None) their indices, the best first.  With `shared_weight` (float32
+    [n]) the router has one row more, whose product's logistic function goes there."""
     n, W = h.shape
-    E = router.shape[0]
+    E = weights.shape[1]
     _req(h, "route.h")
-    _req(router, "route.router", torch.float32, (E, W))
+    _req(router, "route.router", torch.float32, (E + (1 if shared_weight is not None else 0), W))
     _req(weights, "route.weights", torch.float32, (n, E))
     if chosen is not None:
         _req(chosen, "route.chosen", torch.int32, (n, top))
+    if correction is not None:
+        _req(correction, "route.correction", torch.float32, (E,))
     _check(lib().tl_route(_p(h), _code(h.dtype), n, W, _p(router), E, int(groups), int(keep), int(top), int(bool(logistic)),
-                          _p(weights), _p(chosen), _stream()))
+                          _p(correction), int(bool(two_largest)), int(normalise_eps is not None),
+                          ctypes.c_float(normalise_eps or 0.0), _shared_weight(shared_weight, n, "route"), _p(weights),
+                          _p(chosen), _stream()))
 
 
 class GateTerms:
     """The constants of a gated expert, act(g, u) = g' logistic(alpha g') (u' + shift) with g' = min(g, limit) and
     u' = clamp(u, -limit, limit); the shared expert has a limit of its own (`limit_shared`; None: the same).
-    `on_input`: the router's weight multiplies the expert's input (g and u before the clamps) instead of its output."""
+    `on_input`: the router's weight multiplies the expert's input (g and u before the clamps) instead of its output.
+    Limits of infinity, alpha 1 and shift 0 make it silu(g) u."""
 
     def __init__(self, limit: float, alpha: float, shift: float, limit_shared: Optional[float] = None, on_input: bool = False):
         self.limit, self.alpha, self.shift = float(limit), float(alpha), float(shift)
@@ -948,23 +982,23 @@ class GateTerms:
 
 
 def expert_gated_act(gu: torch.Tensor, weights: Optional[torch.Tensor], E: int, ff: int, shared: int, terms: GateTerms,
-                     out: torch.Tensor) -> None:
+                     out: torch.Tensor, shared_weight: Optional[torch.Tensor] = None) -> None:
     """The activations of gated experts laid side by side: gu float32 [n, 2 (E ff + shared)] holds, expert after
     expert, [gate (ff) | up (ff)] and behind them the shared expert's [gate (shared) | up (shared)]; out
     [n, E ff + shared] = act(g, u) with the row's weight of the column's expert (`weights` float32 [n, E]; the
-    shared part has weight 1; E 0: no weights)."""
+    shared part has weight 1, or `shared_weight` float32 [n] on its output; E 0: no weights)."""
     n = gu.shape[0]
     total = E * ff + shared
     _req(gu, "expert_gated_act.gu", torch.float32, (n, 2 * total))
     if E:
         _req(weights, "expert_gated_act.weights", torch.float32, (n, E))
     _req(out, "expert_gated_act.out", None, (n, total))
-    _check(lib().tl_expert_gated_act(_p(gu), _p(weights) if E else None, n, int(E), int(ff), int(shared), *terms.args(),
+    _check(lib().tl_expert_gated_act(_p(gu), _p(weights) if E else None, _shared_weight(shared_weight, n, "expert_gated_act"), n, int(E), int(ff), int(shared), *terms.args(),
                                      _p(out), _code(out.dtype), _stream()))
 
 
 def expert_rows_gated_up(y: torch.Tensor, up: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, ff: int, shared: int,
-                         terms: GateTerms, hs: torch.Tensor) -> None:
+                         terms: GateTerms, hs: torch.Tensor, shared_weight: Optional[torch.Tensor] = None) -> None:
     """The chosen gated experts' first halves, row by row (see `expert_rows_up`): up [2 (E ff + shared), H] is the
     stacked matrix of `expert_gated_act`'s layout."""
     n, H = y.shape
@@ -974,38 +1008,40 @@ def expert_rows_gated_up(y: torch.Tensor, up: torch.Tensor, chosen: torch.Tensor
     _req(chosen, "expert_rows_gated_up.chosen", torch.int32, (n, top))
     _req(weights, "expert_rows_gated_up.weights", torch.float32, (n, E))
     _req(hs, "expert_rows_gated_up.hs", y.dtype, (n, top * ff + shared))
-    _check(lib().tl_expert_rows_gated_up(_p(y), H, _p(up), _p(chosen), _p(weights), n, E, top, int(ff), int(shared),
+    _check(lib().tl_expert_rows_gated_up(_p(y), H, _p(up), _p(chosen), _p(weights),
+                                         _shared_weight(shared_weight, n, "expert_rows_gated_up"), n, E, top, int(ff), int(shared),
                                          *terms.args(), _p(hs), _code(y.dtype), _stream()))
 
 
-def expert_act(u: torch.Tensor, weights: Optional[torch.Tensor], E: int, ff: int, activation: str, out: torch.Tensor) -> None:
-    """out[n, j] = act(u[n, j]) * (weights[n, j // ff] for the first E * ff columns, 1 for the rest); u float32."""
+def expert_act(u: torch.Tensor, weights: Optional[torch.Tensor], E: int, ff: int, activation: str, out: torch.Tensor,
+               constants=None, shared_weight: Optional[torch.Tensor] = None) -> None:
+    """out[n, j] = act(u[n, j]) * (weights[n, j // ff] for the first E * ff columns, 1 or `shared_weight[n]` for the
+    rest); u float32; `constants` by name for an activation of `UNARY_CONSTANTS`."""
     n, total = u.shape
-    if activation not in EXPERT_ACTIVATIONS:
-        raise KernelError(f"expert_act: no function {activation!r}; there are {sorted(EXPERT_ACTIVATIONS)}")
+    code = _unary_args(activation, constants)
     _req(u, "expert_act.u", torch.float32)
     if E:
         _req(weights, "expert_act.weights", torch.float32, (n, E))
     _req(out, "expert_act.out", None, (n, total))
-    _check(lib().tl_expert_act(_p(u), _p(weights) if E else None, n, int(E), int(ff), total, EXPERT_ACTIVATIONS[activation],
+    _check(lib().tl_expert_act(_p(u), _p(weights) if E else None, _shared_weight(shared_weight, n, "expert_act"), n, int(E),
+                               int(ff), total, *code,
                                _p(out), _code(out.dtype), _stream()))
 
 
 def expert_rows_up(y: torch.Tensor, up: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, ff: int, shared: int,
-                   activation: str, hs: torch.Tensor) -> None:
+                   activation: str, hs: torch.Tensor, constants=None, shared_weight: Optional[torch.Tensor] = None) -> None:
     """The chosen experts' first halves, row by row: hs[n, k*ff + j] = act(up[chosen[n,k]*ff + j] . y[n]) * weights[n, chosen[n,k]]
-    and, behind them, the shared expert's `shared` rows with weight 1.  up [E*ff + shared, H] and y [n, H] of one dtype."""
+    and, behind them, the shared expert's `shared` rows with weight 1 (or `shared_weight[n]`).  up [E*ff + shared, H] and y [n, H] of one dtype."""
     n, H = y.shape
     top, E = chosen.shape[1], weights.shape[1]
-    if activation not in EXPERT_ACTIVATIONS:
-        raise KernelError(f"expert_rows_up: no function {activation!r}; there are {sorted(EXPERT_ACTIVATIONS)}")
+    code = _unary_args(activation, constants)
     _req(y, "expert_rows_up.y")
     _req(up, "expert_rows_up.up", y.dtype, (E * ff + shared, H))
     _req(chosen, "expert_rows_up.chosen", torch.int32, (n, top))
     _req(weights, "expert_rows_up.weights", torch.float32, (n, E))
     _req(hs, "expert_rows_up.hs", y.dtype, (n, top * ff + shared))
-    _check(lib().tl_expert_rows_up(_p(y), H, _p(up), _p(chosen), _p(weights), n, E, top, int(ff), int(shared),
-                                   EXPERT_ACTIVATIONS[activation], _p(hs), _code(y.dtype), _stream()))
+    _check(lib().tl_expert_rows_up(_p(y), H, _p(up), _p(chosen), _p(weights), _shared_weight(shared_weight, n, "expert_rows_up"),
+                                   n, E, top, int(ff), int(shared), *code, _p(hs), _code(y.dtype), _stream()))
 
 
 def expert_rows_down(hs: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor, E: int, ff: int, shared: int, out: torch.Tensor,
@@ -1021,6 +1057,190 @@ def expert_rows_down(hs: torch.Tensor, down: torch.Tensor, chosen: torch.Tensor,
     _req(out, "expert_rows_down.out", torch.float32, (n, H))
     _check(lib().tl_expert_rows_down(_p(hs), _p(down), _p(chosen), n, int(E), top, int(ff), int(shared), H, int(bool(accumulate)),
                                      _p(out), _code(hs.dtype), _stream()))
+
+
+# ---- attention over cached latents ---------------------------------------------------------------------
+LATENT_MAX_R, LATENT_MAX_ROT = 1024, 256
+
+
+def _req_latent_pages(pages: torch.Tensor, D: int, dtype, what: str) -> None:
+    _req(pages, what + ".pages", dtype)
+    if pages.dim() < 2 or pages.numel() != pages.shape[0] * PAGE * D:
+        raise KernelError(f"{what}.pages: shape {tuple(pages.shape)}, kernel needs {PAGE} rows of {D} a page")
+
+
+def _req_table(table: torch.Tensor, B: int, what: str) -> int:
+    _req(table, what + ".table", torch.int32)
+    if table.dim() != 2 or table.shape[0] != B:
+        raise KernelError(f"{what}.table: needs one row per sequence")
+    return table.shape[1]
+
+
+def latent_prepare(qf: torch.Tensor, cf: torch.Tensor, row_pos, rotation, H: int, dn: int, dr: int, w: torch.Tensor, eps: float,
+                   qn: torch.Tensor, qr: Optional[torch.Tensor], c: Optional[torch.Tensor], rows: Optional[torch.Tensor],
+                   table=None, ring_pages: int = 0, pages=None) -> None:
+    """One pass over the products of an attention out of latents.  qf float32 [n, H * (dn + dr)] and cf float32
+    [n, R + dr] (both may be columns of wider rows: stride(1) 1) -> qn [n, H, dn], qr [n, H, dr] (rotated;
+    both may be strided views with stride(2) 1), c [n, R] = the normed latent (or None) and rows [n, R + dr] = [c | rotated
+    key part] (or None), or with `pages` (one token a sequence, row n belongs to sequence n) that row straight into
+    the page of its position."""
+    n, R = qf.shape[0], w.shape[0]
+    rot = _rotation(rotation, dr, "latent_prepare", magnitude=True)
+    for t, width, name in ((qf, H * (dn + dr), "qf"), (cf, R + dr, "cf")):
+        if not t.is_cuda or t.dtype != torch.float32 or t.dim() != 2 or tuple(t.shape) != (n, width) or t.stride(1) != 1:
+            raise KernelError(f"latent_prepare.{name}: float32 [{n}, {width}] on the GPU, rows may be strided")
+    _req(w, "latent_prepare.w", torch.float32, (R,))
+    _req(row_pos, "latent_prepare.row_pos", torch.int32, (n,))
+    dt = qn.dtype
+    for t, width, name in ((qn, dn, "qn"),) + (((qr, dr, "qr"),) if dr else ()):
+        if t is None or not t.is_cuda or t.dtype != dt or tuple(t.shape) != (n, H, width) or t.stride(2) != 1:
+            raise KernelError(f"latent_prepare.{name}: [{n}, {H}, {width}] on the GPU, heads may be strided")
+    if c is not None:
+        _req(c, "latent_prepare.c", dt, (n, R))
+    if rows is not None:
+        _req(rows, "latent_prepare.rows", dt, (n, R + dr))
+    stride = 0
+    if pages is not None:
+        _req_latent_pages(pages, R + dr, dt, "latent_prepare")
+        stride = _req_table(table, n, "latent_prepare")
+    L = ctypes.c_longlong
+    _check(lib().tl_latent_prepare(_p(qf), qf.stride(0), _p(cf), cf.stride(0), n, H, dn, dr, R, _p(w), ctypes.c_float(eps),
+                                   _p(row_pos), _p(rot.inv_freq), rot.rotary_dim, int(rot.interleaved),
+                                   ctypes.c_float(rot.magnitude), _p(qn), L(qn.stride(0)), L(qn.stride(1)),
+                                   _p(qr) if dr else None, L(qr.stride(0) if dr else 0), L(qr.stride(1) if dr else 0), _p(c),
+                                   _p(rows), _p(pages), _p(table) if pages is not None else None, stride, int(ring_pages),
+                                   _code(dt), _stream()))
+
+
+def latent_commit(rows: torch.Tensor, row_seq, row_pos, len_after, table: torch.Tensor, ring_pages: int, pages: torch.Tensor) -> None:
+    """Rows [n, D] into the pages of their positions."""
+    n, D = rows.shape
+    _req(rows, "latent_commit.rows")
+    _req_latent_pages(pages, D, rows.dtype, "latent_commit")
+    _req(row_seq, "latent_commit.row_seq", torch.int32, (n,))
+    _req(row_pos, "latent_commit.row_pos", torch.int32, (n,))
+    B = len_after.shape[0]
+    _req(len_after, "latent_commit.len_after", torch.int32, (B,))
+    stride = _req_table(table, B, "latent_commit")
+    _check(lib().tl_latent_commit(_p(rows), _code(rows.dtype), _p(row_seq), _p(row_pos), _p(len_after), _p(table), stride,
+                                  int(ring_pages), n, D, _p(pages), _stream()))
+
+
+def latent_gather(pages: torch.Tensor, table: torch.Tensor, off: torch.Tensor, n_pages: int, c: torch.Tensor,
+                  kr: Optional[torch.Tensor]) -> None:
+    """The pages of a step's sequences one behind the other: off int32 [B + 1] is the running number of pages, of
+    sequence b's the first off[b + 1] - off[b] entries of its row of `table`; c [n_pages * 64, R], kr [n_pages * 64, dr]."""
+    R, dr = c.shape[1], 0 if kr is None else kr.shape[1]
+    B = table.shape[0]
+    _req_latent_pages(pages, R + dr, c.dtype, "latent_gather")
+    stride = _req_table(table, B, "latent_gather")
+    _req(off, "latent_gather.off", torch.int32, (B + 1,))
+    _req(c, "latent_gather.c", None, (n_pages * PAGE, R))
+    if dr:
+        _req(kr, "latent_gather.kr", c.dtype, (n_pages * PAGE, dr))
+    _check(lib().tl_latent_gather(_p(pages), _code(c.dtype), _p(table), stride, _p(off), B, int(n_pages), R, dr, _p(c), _p(kr),
+                                  _stream()))
+
+
+def latent_heads(kvf: torch.Tensor, kr: Optional[torch.Tensor], H: int, dn: int, dr: int, dv: int, k: torch.Tensor,
+                 v: torch.Tensor) -> None:
+    """kvf float32 [n, H * (dn + dv)] = [keys of all heads | values of all heads] and kr [n, dr] (rows may be strided) ->
+    k [n, H, dn + dr] with the shared part behind every head's own, v [n, H, dv]."""
+    n = kvf.shape[0]
+    _req(kvf, "latent_heads.kvf", torch.float32, (n, H * (dn + dv)))
+    _req(k, "latent_heads.k", None, (n, H, dn + dr))
+    _req(v, "latent_heads.v", k.dtype, (n, H, dv))
+    if dr and (kr.dtype != k.dtype or tuple(kr.shape) != (n, dr) or kr.stride(1) != 1 or not kr.is_cuda):
+        raise KernelError(f"latent_heads.kr: [{n}, {dr}] of k's dtype on the GPU, rows may be strided")
+    _check(lib().tl_latent_heads(_p(kvf), _p(kr) if dr else None, kr.stride(0) if dr else 0, n, H, dn, dr, dv, _p(k), _p(v),
+                                 _code(k.dtype), _stream()))
+
+
+def latent_heads_pages(kvf: torch.Tensor, kr: Optional[torch.Tensor], H: int, dn: int, dr: int, dv: int, pages: torch.Tensor) -> None:
+    """`latent_heads` of gathered pages: kvf float32 [n_pages * 64, H * (dn + dv)], kr [n_pages * 64, dr] -> pages as
+    `KVGroup` keeps keys and values per head."""
+    n = pages.shape[0]
+    _req(kvf, "latent_heads_pages.kvf", torch.float32, (n * PAGE, H * (dn + dv)))
+    if dr:
+        _req(kr, "latent_heads_pages.kr", pages.dtype, (n * PAGE, dr))
+    _req_pages(pages, H, dn + dr, dv, "latent_heads_pages")
+    _check(lib().tl_latent_heads_pages(_p(kvf), _p(kr) if dr else None, n, H, dn, dr, dv, _p(pages), _code(pages.dtype), _stream()))
+
+
+def head_products(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> None:
+    """out[n, h] = w[h] x[n, h] for every head: x [n, H, K], w [H, N, K] and out [n, H, N] (heads may be strided) of one
+    dtype, float32 sums."""
+    n, H, K = x.shape
+    N = w.shape[1]
+    _req(x, "head_products.x")
+    _req(w, "head_products.w", x.dtype, (H, N, K))
+    if out.dtype != x.dtype or tuple(out.shape) != (n, H, N) or out.stride(2) != 1 or not out.is_cuda:
+        raise KernelError(f"head_products.out: [{n}, {H}, {N}] of x's dtype on the GPU, heads may be strided")
+    _check(lib().tl_head_products(_p(x), _p(w), n, H, N, K, _p(out), ctypes.c_longlong(out.stride(0)),
+                                  ctypes.c_longlong(out.stride(1)), _code(x.dtype), _stream()))
+
+
+def latent_attention(q: torch.Tensor, pages: torch.Tensor, table: torch.Tensor, ring_pages: int, ctx, dr: int,
+                     window: Optional[int], scale: float, out: torch.Tensor) -> None:
+    """Attention of one token a sequence over its cached rows [c | k_r] (its own is committed): q [B, H, R + dr] in the
+    rows' channels, out [B, H, R] = the softmax-weighted sum of c."""
+    B, H, D = q.shape
+    R = D - dr
+    _req(q, "latent_attention.q")
+    _req_latent_pages(pages, D, q.dtype, "latent_attention")
+    stride = _req_table(table, B, "latent_attention")
+    _req(ctx.row_pos, "latent_attention.row_pos", torch.int32, (B,))
+    _req(out, "latent_attention.out", q.dtype, (B, H, R))
+    _check(lib().tl_latent_attn_plain(_p(q), _p(pages), _code(q.dtype), _p(table), stride, int(ring_pages), _p(ctx.row_pos), B, H, R,
+                                      dr, int(window or 0), ctypes.c_float(scale), _p(out), _stream()))
+
+
+def attend_heads(ctx, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, pages: torch.Tensor, table: torch.Tensor,
+                 ring_pages: int, terms: "ScoreTerms", out: torch.Tensor) -> None:
+    """Attention of a step's rows over their own keys and values (k [n, H, dk], v [n, H, dv]) and, for cached positions,
+    those of `pages` (flat, of the kind that `KVGroup` keeps), nothing committed."""
+    H, dv = k.shape[1], v.shape[2]
+    attn_scored_plain(q, k, v, pages, H, dv, table, ring_pages, ctx.row_seq, ctx.row_pos, ctx.cu_seqlens, ctx.len_before,
+                      terms, None, out)
+
+
+# ---- retention -----------------------------------------------------------------------------------------
+def _req_state(state: torch.Tensor, elems: int, what: str) -> None:
+    if state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1 or not state.is_cuda or state.shape[1] < elems:
+        raise KernelError(f"{what}.state: float32 [slots, {elems} or more] on the GPU, rows may be strided")
+
+
+def retention_scan(proj: torch.Tensor, row_pos, rotation, H: int, dk: int, dv: int, kscale: float, decay: torch.Tensor,
+                   state: torch.Tensor, cu_seqlens, slots, o: torch.Tensor) -> None:
+    """Row after row, sequence by sequence, all in float32: proj [n, width] starts with [q | k | v] (H heads of dk, dk,
+    dv); q and k rotated, k times kscale; S <- decay[h] S + k v^T, o = S^T q; `state` float32 [slots, >= H*dk*dv] is read
+    and left updated; o float32 [n, H*dv]."""
+    n, width = proj.shape
+    B = slots.shape[0]
+    rot = _rotation(rotation, dk, "retention", magnitude=True)
+    _req(proj, "retention.proj", torch.float32)
+    _req(row_pos, "retention.row_pos", torch.int32, (n,))
+    _req(decay, "retention.decay", torch.float32, (H,))
+    _req_state(state, H * dk * dv, "retention")
+    _req(cu_seqlens, "retention.cu_seqlens", torch.int32, (B + 1,))
+    _req(slots, "retention.slots", torch.int32)
+    _req(o, "retention.o", torch.float32, (n, H * dv))
+    _check(lib().tl_retention_scan(_p(proj), width, H, dk, dv, _p(row_pos), _p(rot.inv_freq), rot.rotary_dim,
+                                   int(rot.interleaved), ctypes.c_float(rot.magnitude), ctypes.c_float(kscale), _p(decay),
+                                   _p(state), ctypes.c_longlong(state.stride(0)), _p(cu_seqlens), _p(slots), n, B, _p(o),
+                                   _stream()))
+
+
+def retention_norm_gate(o: torch.Tensor, gate: torch.Tensor, H: int, eps: float, out: torch.Tensor) -> None:
+    """out[n, h] = o / sqrt(mean(o^2) + eps) * silu(gate) per head: o float32 [n, H*dv], gate float32 [n, H*dv] (rows may
+    be strided: columns of the projection), out in the compute dtype."""
+    n, inner = o.shape
+    _req(o, "retention_norm_gate.o", torch.float32)
+    if gate.dtype != torch.float32 or tuple(gate.shape) != (n, inner) or gate.stride(1) != 1 or not gate.is_cuda:
+        raise KernelError(f"retention_norm_gate.gate: float32 [{n}, {inner}] on the GPU, rows may be strided")
+    _req(out, "retention_norm_gate.out", None, (n, inner))
+    _check(lib().tl_retention_norm_gate(_p(o), _p(gate), gate.stride(0), n, H, inner // H, ctypes.c_float(eps), _p(out),
+                                        _code(out.dtype), _stream()))
 
 
 def take_tokens(src: torch.Tensor, idx: torch.Tensor, vocab: int, tokens: torch.Tensor) -> None:

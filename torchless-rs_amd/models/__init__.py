@@ -8,6 +8,7 @@ from . import sozetar as _sozetar         # registers Sozetar
 from . import fanitar as _fanitar         # registers Fanitar
 from . import nepisun as _nepisun         # registers Nepisun
 from . import giforax as _giforax         # registers Giforax
+from . import zudalorn as _zudalorn       # registers Zudalorn
 
 
 def model_spec_for(cfg: ModelConfig):

@@ -18,18 +18,20 @@ class RMSNorm(Norm):
     graph_safe = True
     takes_pending = True        # adds partial products left in ctx.pending while it reads the stream
 
-    def __init__(self, size: int, eps: float, name: str = "weight"):
-        """`name`: the weight's leaf name behind the norm's prefix ("" where the prefix is the tensor)."""
+    def __init__(self, size: int, eps: float, name: str = "weight", scalar: bool = False):
+        """`name`: the weight's leaf name behind the norm's prefix ("" where the prefix is the tensor);
+        `scalar`: the weight is one number for all channels (a tensor without dimensions)."""
         self.size = int(size)
         self.eps = float(eps)
         self.name = name
+        self.scalar = bool(scalar)
         self.weight = None
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
-        return {self.name: WeightSpec((self.size,), init="ones")}
+        return {self.name: WeightSpec(() if self.scalar else (self.size,), init="ones")}
 
     def load(self, tensors, compute_dtype) -> None:
-        self.weight = tensors[self.name].to(torch.float32).contiguous()
+        self.weight = tensors[self.name].to(torch.float32).expand(self.size).contiguous()
 
     def add_to(self, ctx, z: torch.Tensor, x: torch.Tensor, out=None, bias=None, then=None) -> None:
         """x += norm(z + bias) in one kernel.  `then` = (norm, buffer): the norm that reads the

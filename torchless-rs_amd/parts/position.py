@@ -6,10 +6,18 @@ is rotated by the angle pos * inv_freq[i].  The reference rotates the whole head
 rotates the first channels only and `interleaved` pairs (2i, 2i+1) instead.
 Angles, cosines and sines are float32.  The table of inverse frequencies is made
 once on the host in float64 and rounded to float32.
+
+`scaling` = {factor, original, fast, slow} stretches the rotation for contexts longer than the
+`original` positions (Peng et al., YaRN: Efficient Context Window Extension of Large Language
+Models): a pair that turns `fast` times or more within `original` positions keeps its frequency,
+one that turns `slow` times or fewer has it divided by `factor`, and between the two (as indices
+of pairs, rounded outwards) a linear ramp leads from the one to the other; cosines and sines
+are multiplied by 0.1 ln(factor) + 1 (`ops.Rotation.magnitude`).
 """
 from __future__ import annotations
 
-from typing import Optional
+import math
+from typing import Dict, Optional
 
 import torch
 
@@ -18,7 +26,13 @@ from .base import Position, register_part
 
 
 class Rotary(Position):
-    def __init__(self, head_dim: int, theta: float, rotary_dim: Optional[int] = None, interleaved: bool = False):
+    SCALING = ("factor", "original", "fast", "slow")
+
+    def __init__(self, head_dim: int, theta: float, rotary_dim: Optional[int] = None, interleaved: bool = False,
+                 scaling: Optional[Dict[str, float]] = None):
+        if scaling is not None and (set(scaling) != set(self.SCALING) or any(not float(v) > 0 for v in scaling.values())):
+            raise ValueError(f"rotary: scaling takes the positive numbers {self.SCALING}, got {scaling}")
+        self.scaling = None if scaling is None else {k: float(v) for k, v in scaling.items()}
         self.head_dim = int(head_dim)
         self.rotary_dim = self.head_dim if rotary_dim is None else int(rotary_dim)
         if self.rotary_dim % 2 or not (0 < self.rotary_dim <= self.head_dim):
@@ -31,12 +45,27 @@ class Rotary(Position):
     def inv_freq_host(self) -> torch.Tensor:
         half = self.rotary_dim // 2
         i = torch.arange(half, dtype=torch.float64)
-        return (1.0 / torch.pow(torch.tensor(self.theta, dtype=torch.float64), i / half)).to(torch.float32)
+        f = 1.0 / torch.pow(torch.tensor(self.theta, dtype=torch.float64), i / half)
+        if self.scaling is not None:
+            lo, hi = self._pair_of(self.scaling["fast"]), self._pair_of(self.scaling["slow"])
+            lo, hi = max(math.floor(lo), 0), min(math.ceil(hi), self.rotary_dim - 1)
+            ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+            f = f / self.scaling["factor"] * ramp + f * (1.0 - ramp)
+        return f.to(torch.float32)
+
+    def _pair_of(self, turns: float) -> float:
+        """The pair (not a whole number) that turns `turns` times within the original positions."""
+        return self.rotary_dim * math.log(self.scaling["original"] / (2.0 * math.pi * turns)) / (2.0 * math.log(self.theta))
+
+    @property
+    def magnitude(self) -> float:
+        return 1.0 if self.scaling is None else 0.1 * math.log(self.scaling["factor"]) + 1.0
 
     def rotation(self, device) -> ops.Rotation:
         key = str(device)
         if key not in self._rotation:
-            self._rotation[key] = ops.Rotation(self.inv_freq_host().to(device), self.rotary_dim, self.interleaved)
+            self._rotation[key] = ops.Rotation(self.inv_freq_host().to(device), self.rotary_dim, self.interleaved,
+                                              self.magnitude)
         return self._rotation[key]
 
     def inv_freq(self, device) -> torch.Tensor:
