@@ -77,7 +77,9 @@ struct PageSpan {
 constexpr int PF_BM = 128, PF_BN = 64, PF_VLD = PF_BN + 4;
 constexpr int PF_PART_HEAD = 4;       // floats before O in a half block's partial result: maximum, sum, two of padding
 
-template <int DPAD, bool LEAN, bool TERMS = false, bool LOGI = false>   // LEAN (d == DPAD, 256 % (DPAD / 8) == 0): whole tiles are fetched the short way
+// LEAN (d == DPAD, 256 % (DPAD / 8) == 0): whole tiles are fetched the short way.  DV > 0: values of another width than
+// keys, dv_arg channels padded to DV (0: as wide as keys).
+template <int DPAD, bool LEAN, bool TERMS = false, bool LOGI = false, int DV = 0>
 __global__ void __launch_bounds__(256, DPAD <= 128 ? 2 : 1)
 attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
                     const bf16* __restrict__ vt_new, int vt_cols, const int* __restrict__ tile_off,
@@ -85,12 +87,16 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
                     int ring_pages, const int* __restrict__ row_pos, const int* __restrict__ cu_seqlens,
                     const int* __restrict__ n_cached, int B, int n_tiles, int nq, int nkv, int d,
                     int window, float scale, bf16* __restrict__ out, const int4* __restrict__ items,
-                    float* __restrict__ part, int part_ways, MoreTerms terms) {
-  constexpr int KB = DPAD / 16, VB = DPAD / 32, KLD = DPAD + 8, CH = DPAD / 8;
-  constexpr int PT = DPAD / 32;        // 16-byte chunks of keys, and of values, per thread and tile
+                    float* __restrict__ part, int part_ways, MoreTerms terms, int dv_arg) {
+  constexpr int DVP = DV > 0 ? DV : DPAD;
+  constexpr int KB = DPAD / 16, VB = DVP / 32, KLD = DPAD + 8, CH = DPAD / 8;
+  constexpr int PT = DPAD / 32;        // 16-byte chunks of keys per thread and tile
+  constexpr int PTV = DVP / 32;        // ... and of values
+  constexpr int PTM = PT > PTV ? PT : PTV;
+  static_assert(!LEAN || DV == 0, "the short way is for values as wide as keys");
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16* Ks = reinterpret_cast<bf16*>(smem);          // [PF_BN][KLD]
-  bf16* Vt = Ks + PF_BN * KLD;                       // [DPAD][PF_VLD]
+  bf16* Vt = Ks + PF_BN * KLD;                       // [DVP][PF_VLD]
 
   // Which head and which block of rows.  Workgroups are dealt round to the 8 XCDs and start in the order
   // of their numbers.  An XCD takes nq / 8 neighbouring heads, whose one or two KV heads stay in its L2,
@@ -140,9 +146,11 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
   const int row0 = cu_seqlens[b], n_new = cu_seqlens[b + 1] - row0;
   const int cached = n_cached[b];
   const int p_first = row_pos[row0];
-  const size_t head_elems = (size_t)PAGE * d, page_elems = 2 * (size_t)nkv * head_elems;
+  const int dv_n = DV > 0 ? dv_arg : d;               // value channels
+  const size_t head_elems = (size_t)PAGE * d, v_elems = DV > 0 ? (size_t)PAGE * dv_n : head_elems;
+  const size_t page_elems = DV > 0 ? (size_t)nkv * (head_elems + v_elems) : 2 * (size_t)nkv * head_elems;
   const int j_base = (cached / PAGE) * PAGE;
-  const bf16* vt_head = vt_new + (size_t)kvh * d * vt_cols + tile_off[b];
+  const bf16* vt_head = vt_new + (size_t)kvh * dv_n * vt_cols + tile_off[b];
   const int seq_end = p_first + n_new;               // one past the sequence's last position
   static_assert(PF_BN == PAGE, "a tile of keys below n_cached is one page");
   static_assert(!LEAN || 256 % CH == 0, "the short way needs every thread's chunks in one column of chunks");
@@ -193,7 +201,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
   if (chunk > 0) j_lo = max(j_lo, (p_lo / chunk) * chunk);
   const int c_lo_me = chunk > 0 ? (p_me / chunk) * chunk : 0;         // the first key of this lane's query's chunk
 
-  bf16x8 kfetch[PT], vfetch[PT];
+  bf16x8 kfetch[PT], vfetch[PTV];
   // tile j0 -> registers: keys as rows [key][d], values as rows [dv][key]
   // Whole tiles of a head that fills its padded size take the short way: the workgroup's base
   // address is uniform and a thread's chunks lie at fixed offsets from it, one stride apart.
@@ -233,18 +241,19 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
     if (j0 + PF_BN <= cached) {
       // a cached page: keys [64][d], values [d][64]
       const bf16* kpage = pages + (size_t)page * page_elems + (size_t)kvh * head_elems;
-      const bf16* vpage = kpage + (size_t)nkv * head_elems;
+      const bf16* vpage = DV > 0 ? pages + (size_t)page * page_elems + (size_t)nkv * head_elems + (size_t)kvh * v_elems
+                                 : kpage + (size_t)nkv * head_elems;
       if constexpr (LEAN) {
         fetch_lean(kpage, 2u * d, vpage, 2u * PAGE);        // rows [64][d] and [d][64]
         return;
       }
 #pragma unroll
-      for (int i = 0; i < PT; ++i) {
+      for (int i = 0; i < PTM; ++i) {
         const int c = tid + 256 * i;
         const int row = c / CH, col = (c % CH) * 8;
-        kfetch[i] = (col < d) ? ld8(kpage + (size_t)row * d + col) : z8();
+        if (i < PT) kfetch[i < PT ? i : 0] = (col < d) ? ld8(kpage + (size_t)row * d + col) : z8();
         const int dv = c / (PF_BN / 8), kc = (c % (PF_BN / 8)) * 8;
-        vfetch[i] = (dv < d) ? ld8(vpage + (size_t)dv * PAGE + kc) : z8();
+        if (i < PTV) vfetch[i < PTV ? i : 0] = (dv < dv_n) ? ld8(vpage + (size_t)dv * PAGE + kc) : z8();
       }
       return;
     }
@@ -257,40 +266,43 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
         return;
       }
 #pragma unroll
-      for (int i = 0; i < PT; ++i) {
+      for (int i = 0; i < PTM; ++i) {
         const int c = tid + 256 * i;
         const int row = c / CH, col = (c % CH) * 8;
-        kfetch[i] = (col < d) ? ld8(krows + (size_t)row * nkv * d + col) : z8();
+        if (i < PT) kfetch[i < PT ? i : 0] = (col < d) ? ld8(krows + (size_t)row * nkv * d + col) : z8();
         const int dv = c / (PF_BN / 8), kc = (c % (PF_BN / 8)) * 8;
-        vfetch[i] = (dv < d) ? ld8(vcols + (size_t)dv * vt_cols + kc) : z8();
+        if (i < PTV) vfetch[i < PTV ? i : 0] = (dv < dv_n) ? ld8(vcols + (size_t)dv * vt_cols + kc) : z8();
       }
       return;
     }
     // the tile that holds the boundary between cached and new rows, or the sequence's end
     const bool has_cached = j0 < cached, has_new = j0 + PF_BN > cached;
     const bf16* kpage = nullptr;
+    const bf16* vpage = nullptr;
     if (has_cached) {
       const int page = table[(size_t)b * table_stride + (j0 / PAGE) % ring_pages];
       kpage = pages + (size_t)page * page_elems + (size_t)kvh * head_elems;
+      vpage = DV > 0 ? pages + (size_t)page * page_elems + (size_t)nkv * head_elems + (size_t)kvh * v_elems
+                     : kpage + (size_t)nkv * head_elems;
     }
 #pragma unroll
-    for (int i = 0; i < PT; ++i) {
+    for (int i = 0; i < PTM; ++i) {
       const int c = tid + 256 * i;
-      {   // keys: chunk c = (row, 8 columns)
+      if (i < PT) {   // keys: chunk c = (row, 8 columns)
         const int row = c / CH, col = (c % CH) * 8, j = j0 + row;
         bf16x8 kv = z8();
         if (col < d && j < seq_end) {
           if (j < cached) kv = ld8(kpage + (size_t)row * d + col);
           else kv = ld8(k_new + ((size_t)(row0 + j - cached) * nkv + kvh) * d + col);
         }
-        kfetch[i] = kv;
+        kfetch[i < PT ? i : 0] = kv;
       }
-      {   // values: chunk c = (dv, 8 keys); columns past the sequence's end were never written
+      if (i < PTV) {   // values: chunk c = (dv, 8 keys); columns past the sequence's end were never written
         const int dv = c / (PF_BN / 8), kc = (c % (PF_BN / 8)) * 8;
         bf16x8 vv = z8();
-        if (dv < d) {
+        if (dv < dv_n) {
           bf16x8 cv = z8(), nv = z8();
-          if (has_cached) cv = ld8(kpage + (size_t)nkv * head_elems + (size_t)dv * PAGE + kc);
+          if (has_cached) cv = ld8(vpage + (size_t)dv * PAGE + kc);
           if (has_new) nv = ld8(vt_head + (size_t)dv * vt_cols + (j0 - j_base) + kc);
 #pragma unroll
           for (int e = 0; e < 8; ++e) {
@@ -298,22 +310,23 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
             vv[e] = (j < cached) ? cv[e] : ((j < seq_end) ? nv[e] : (bf16)0.f);
           }
         }
-        vfetch[i] = vv;
+        vfetch[i < PTV ? i : 0] = vv;
       }
     }
   };
   auto stash = [&]() {
 #pragma unroll
-    for (int i = 0; i < PT; ++i) {
+    for (int i = 0; i < PTM; ++i) {
       const int c = tid + 256 * i;
       const int row = c / CH, col = (c % CH) * 8;
-      *reinterpret_cast<bf16x8*>(&Ks[row * KLD + col]) = kfetch[i];
+      if (i < PT) *reinterpret_cast<bf16x8*>(&Ks[row * KLD + col]) = kfetch[i < PT ? i : 0];
+      if (i >= PTV) continue;
       const int dv = c / (PF_BN / 8), kc = (c % (PF_BN / 8)) * 8;
       bf16x4 lo4, hi4;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        lo4[e] = vfetch[i][e];
-        hi4[e] = vfetch[i][4 + e];
+        lo4[e] = vfetch[i < PTV ? i : 0][e];
+        hi4[e] = vfetch[i < PTV ? i : 0][4 + e];
       }
       *reinterpret_cast<bf16x4*>(&Vt[dv * PF_VLD + kc]) = lo4;
       *reinterpret_cast<bf16x4*>(&Vt[dv * PF_VLD + kc + 4]) = hi4;
@@ -451,7 +464,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
   if (ways != 0) {
     // a run of a block's keys: running maximum, sum and unscaled O of every row, for the merge
     if (q_ok) {
-      float* pp = part + (((size_t)(row0 + qr) * nq + h) * part_ways + slot) * (size_t)(d + PF_PART_HEAD);
+      float* pp = part + (((size_t)(row0 + qr) * nq + h) * part_ways + slot) * (size_t)(dv_n + PF_PART_HEAD);
       if (half == 0) {
         pp[0] = m;
         pp[1] = l;
@@ -461,7 +474,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
 #pragma unroll
         for (int g4 = 0; g4 < 4; ++g4) {                 // four values in a row: 16 bytes a store
           const int dv = vb * 32 + 8 * g4 + 4 * half;
-          if (dv < d)
+          if (dv < dv_n)
             *reinterpret_cast<f32x4*>(pp + PF_PART_HEAD + dv) =
                 f32x4{o[vb][4 * g4], o[vb][4 * g4 + 1], o[vb][4 * g4 + 2], o[vb][4 * g4 + 3]};
         }
@@ -469,7 +482,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
     return;
   }
   if (q_ok) {
-    bf16* op = out + ((size_t)(row0 + qr) * nq + h) * d;
+    bf16* op = out + ((size_t)(row0 + qr) * nq + h) * dv_n;
     float inv = 1.0f / l;
     if constexpr (TERMS)
       if (terms.gate != nullptr) inv *= terms.gate[(size_t)(row0 + qr) * nq + h];
@@ -478,7 +491,7 @@ attn_prefill_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k_new,
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int dv = vb * 32 + 8 * (r / 4) + 4 * half + (r % 4);
-        if (dv < d) op[dv] = (bf16)(o[vb][r] * inv);
+        if (dv < dv_n) op[dv] = (bf16)(o[vb][r] * inv);
       }
   }
 }
@@ -1105,12 +1118,12 @@ static int launch_prefill_v(const bf16* q, const bf16* k_new, const bf16* vt_new
     attn_prefill_kernel<DPAD, can_lean, TERMS, LOGI><<<grid, 256, smem, st>>>(q, k_new, vt_new, vt_cols, tile_off, pages, table,
                                                              table_stride, ring_pages, row_pos, cu_seqlens,
                                                              n_cached, B, n_tiles, nq, nkv, d, window, scale, out,
-                                                             items, part, part_ways, terms);
+                                                             items, part, part_ways, terms, d);
   else
     attn_prefill_kernel<DPAD, false, TERMS, LOGI><<<grid, 256, smem, st>>>(q, k_new, vt_new, vt_cols, tile_off, pages, table,
                                                               table_stride, ring_pages, row_pos, cu_seqlens,
                                                               n_cached, B, n_tiles, nq, nkv, d, window, scale, out,
-                                                              items, part, part_ways, terms);
+                                                              items, part, part_ways, terms, d);
   TL_LAUNCH_CHECK("attn_prefill");
   if (n_cut > 0) {
     const int pieces = (PF_BM * d + PF_MERGE - 1) / PF_MERGE;
@@ -1140,6 +1153,43 @@ static int launch_prefill(const bf16* q, const bf16* k_new, const bf16* vt_new, 
   return launch_prefill_v<DPAD, false>(q, k_new, vt_new, vt_cols, tile_off, pages, table, table_stride, ring_pages,
                                        row_pos, cu_seqlens, n_cached, B, n_tiles, nq, nkv, d, window, scale, out,
                                        items, cut_blocks, n_cut, part, part_ways, st, MoreTerms{});
+}
+
+// plain scores, values of another width than keys
+template <int DPAD, int DV>
+static int launch_prefill_wide(const bf16* q, const bf16* k_new, const bf16* vt_new, int vt_cols, const int* tile_off,
+                               const bf16* pages, const int* table, int table_stride, int ring_pages, const int* row_pos,
+                               const int* cu_seqlens, const int* n_cached, int B, int n_tiles, int nq, int nkv, int dk, int dv,
+                               int window, float scale, bf16* out, const int4* items, const int4* cut_blocks, int n_cut,
+                               float* part, int part_ways, hipStream_t st) {
+  const size_t smem = ((size_t)PF_BN * (DPAD + 8) + (size_t)DV * PF_VLD) * sizeof(bf16);
+  if (smem > 48 * 1024) {
+    static bool raised = false;
+    if (!raised) {
+      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&attn_prefill_kernel<DPAD, false, false, false, DV>),
+                                               hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem);
+      if (e != hipSuccess) {
+        set_error("attn_prefill: cannot have %zu bytes of LDS: %s", smem, hipGetErrorString(e));
+        return 2;
+      }
+      raised = true;
+    }
+  }
+  const long long total = (long long)n_tiles * nq;
+  if (total > 2147483000LL) {
+    set_error("attn_prefill: %lld (head, block of rows) pairs are too many", total);
+    return 1;
+  }
+  attn_prefill_kernel<DPAD, false, false, false, DV><<<(unsigned)total, 256, smem, st>>>(
+      q, k_new, vt_new, vt_cols, tile_off, pages, table, table_stride, ring_pages, row_pos, cu_seqlens, n_cached, B, n_tiles, nq,
+      nkv, dk, window, scale, out, items, part, part_ways, MoreTerms{}, dv);
+  TL_LAUNCH_CHECK("attn_prefill with values of another width");
+  if (n_cut > 0) {
+    const int pieces = (PF_BM * dv + PF_MERGE - 1) / PF_MERGE;
+    attn_prefill_merge_kernel<<<dim3(n_cut * pieces, nq), 256, 0, st>>>(part, part_ways, cut_blocks, cu_seqlens, pieces, nq, dv, out);
+    TL_LAUNCH_CHECK("attn_prefill_merge");
+  }
+  return 0;
 }
 
 // which decode kernel serves head sizes 64, 128 and 256 (tests and measurements may switch)
@@ -1335,6 +1385,46 @@ extern "C" int tl_attn_prefill_terms_bf16(const void* q, const void* k_new, cons
   return attn_prefill_entry(q, k_new, vt_new, vt_cols, tile_off, pages, table, table_stride, ring_pages, row_pos,
                             cu_seqlens, n_cached, B, n_tiles, nq, nkv, d, window, scale, out, nullptr, nullptr, 0,
                             nullptr, 0, 0, 0, st, &terms);
+}
+
+// The same with values of another width than keys: k_new [rows, nkv, dk], vt_new [nkv][dv][vt_cols], a page
+// [keys [nkv][64][dk] | values [nkv][dv][64]], out [rows, nq, dv].
+extern "C" int tl_attn_prefill_wide_bf16(const void* q, const void* k_new, const void* vt_new, int vt_cols,
+                                         const int* tile_off, const void* pages, const int* table, int table_stride,
+                                         int ring_pages, const int* row_pos, const int* cu_seqlens,
+                                         const int* n_cached, int B, int n_tiles, int nq, int nkv, int dk, int dv,
+                                         int window, float scale, void* out, const int* items, const int* cut_blocks,
+                                         int n_cut, float* part, int part_ways, long long part_floats, int n_rows,
+                                         hipStream_t st) {
+  TL_REQUIRE(B > 0 && n_tiles > 0 && nq > 0 && nkv > 0 && nq % nkv == 0 && nq <= 65535,
+             "attn_prefill: bad sizes B=%d tiles=%d nq=%d nkv=%d", B, n_tiles, nq, nkv);
+  TL_REQUIRE(n_cut >= 0 && (n_cut == 0 || (items != nullptr && cut_blocks != nullptr && part != nullptr && n_rows > 0 &&
+                                          part_ways >= 2 && part_ways <= PF_MAX_WAYS &&
+                                          part_floats >= (long long)n_rows * nq * part_ways * (dv + PF_PART_HEAD))),
+             "attn_prefill: %d blocks cut %d ways at most need the entries, the blocks and room for their sums", n_cut, part_ways);
+  TL_REQUIRE(((uintptr_t)items % 16 == 0) && ((uintptr_t)cut_blocks % 16 == 0) && ((uintptr_t)part % 16 == 0),
+             "attn_prefill: the entries and the room for the sums must be 16-byte aligned");
+  TL_REQUIRE(dk >= 8 && dk <= 256 && dk % 8 == 0 && dv >= 4 && dv <= 256 && dv % 4 == 0,
+             "attn_prefill: head sizes %d and %d are not served (keys in multiples of 8, values of 4, up to 256)", dk, dv);
+  TL_REQUIRE(((uintptr_t)q % 16 == 0) && ((uintptr_t)k_new % 16 == 0) && ((uintptr_t)pages % 16 == 0),
+             "attn_prefill: queries, keys and pages must be 16-byte aligned");
+  TL_REQUIRE(ring_pages > 0 && table_stride > 0 && window >= 0, "attn_prefill: bad cache geometry ring_pages=%d table_stride=%d window=%d",
+             ring_pages, table_stride, window);
+  TL_REQUIRE(vt_cols > 0 && vt_cols % 64 == 0 && ((uintptr_t)vt_new % 16 == 0),
+             "attn_prefill: the transposed values need a multiple of 64 columns (%d) and 16-byte alignment", vt_cols);
+#define TL_WIDE(DP, DVP)                                                                                                       \
+  return launch_prefill_wide<DP, DVP>((const bf16*)q, (const bf16*)k_new, (const bf16*)vt_new, vt_cols, tile_off,              \
+                                      (const bf16*)pages, table, table_stride, ring_pages, row_pos, cu_seqlens, n_cached, B,   \
+                                      n_tiles, nq, nkv, dk, dv, window, scale, (bf16*)out, reinterpret_cast<const int4*>(items), \
+                                      reinterpret_cast<const int4*>(cut_blocks), n_cut, part, part_ways, st)
+  if (dk <= 64 && dv <= 64) TL_WIDE(64, 64);
+  if (dk <= 64 && dv <= 128) TL_WIDE(64, 128);
+  if (dk <= 96 && dv <= 64) TL_WIDE(96, 64);
+  if (dk <= 128 && dv <= 128) TL_WIDE(128, 128);
+  if (dk <= 192 && dv <= 128) TL_WIDE(192, 128);
+  if (dk <= 192 && dv <= 192) TL_WIDE(192, 192);
+  TL_WIDE(256, 256);
+#undef TL_WIDE
 }
 
 // For tests and measurements: 1 (the default) lets head sizes 64, 128 and 256 go through the kernel that stages the

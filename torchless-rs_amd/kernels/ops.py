@@ -1176,8 +1176,36 @@ def head_products(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> None:
     _req(w, "head_products.w", x.dtype, (H, N, K))
     if out.dtype != x.dtype or tuple(out.shape) != (n, H, N) or out.stride(2) != 1 or not out.is_cuda:
         raise KernelError(f"head_products.out: [{n}, {H}, {N}] of x's dtype on the GPU, heads may be strided")
-    _check(lib().tl_head_products(_p(x), _p(w), n, H, N, K, _p(out), ctypes.c_longlong(out.stride(0)),
-                                  ctypes.c_longlong(out.stride(1)), _code(x.dtype), _stream()))
+    rest = (_p(x), _p(w), n, H, N, K, _p(out), ctypes.c_longlong(out.stride(0)), ctypes.c_longlong(out.stride(1)))
+    if x.dtype == torch.bfloat16 and K % 8 == 0:
+        _check(lib().tl_head_products_bf16(*rest, compute_units(x.device), _stream()))
+    else:
+        _check(lib().tl_head_products(*rest, _code(x.dtype), _stream()))
+
+
+def latents_on_matrix_cores(dtype: torch.dtype, R: int, dr: int) -> bool:
+    """Does `latent_attention` run on the matrix cores (bfloat16, latents up to 512 channels, rows up to 576 in steps of 8)?"""
+    return dtype == torch.bfloat16 and R <= 512 and R + dr <= 576 and (R + dr) % 8 == 0
+
+
+@functools.lru_cache(maxsize=4096)
+def latent_splits(B: int, H: int, R: int, max_pages: int, units: int):
+    """(head groups of 16 that a workgroup takes, splits of the pages): a workgroup stages a page once for all its heads, so
+    the more heads the fewer bytes, unless compute units stand idle for it; splits as `decode_splits` weighs them."""
+    groups = -(-H // 16)
+    per_unit = 1 if R > 256 else 2                    # a page's rows fill half of a compute unit's LDS, or more
+    room = units * per_unit
+    best = None
+    for hg in (1, 2, 4):
+        if hg > 1 and hg >= 2 * groups:
+            break
+        wide = B * -(-groups // hg)
+        step = 1.0 + 0.25 * (hg - 1)                  # what a page costs with more heads on it
+        for s in range(1, max_pages + 1):
+            cost = -(-wide * s // room) * -(-max_pages // s) * step + SPLIT_COST * s
+            if best is None or cost < best[0] - 1e-9:
+                best = (cost, hg, s)
+    return best[1], best[2]
 
 
 def latent_attention(q: torch.Tensor, pages: torch.Tensor, table: torch.Tensor, ring_pages: int, ctx, dr: int,
@@ -1191,17 +1219,60 @@ def latent_attention(q: torch.Tensor, pages: torch.Tensor, table: torch.Tensor, 
     stride = _req_table(table, B, "latent_attention")
     _req(ctx.row_pos, "latent_attention.row_pos", torch.int32, (B,))
     _req(out, "latent_attention.out", q.dtype, (B, H, R))
+    if latents_on_matrix_cores(q.dtype, R, dr):
+        most = stride if not window else min(stride, -(-window // PAGE) + 1)
+        hg, splits = latent_splits(B, H, R, min(most, 4096), compute_units(q.device))     # (by the table's width: fixed while a graph lives)
+        part = ctx.workspace.get("latent_part", (B * H * splits * (R + 2),), torch.float32) if splits > 1 else None
+        _check(lib().tl_latent_decode_bf16(_p(q), _p(pages), _p(table), stride, int(ring_pages), _p(ctx.row_pos), B, H, R, dr,
+                                           int(window or 0), ctypes.c_float(scale), hg, splits, _p(part), _p(out), _stream()))
+        return
     _check(lib().tl_latent_attn_plain(_p(q), _p(pages), _code(q.dtype), _p(table), stride, int(ring_pages), _p(ctx.row_pos), B, H, R,
                                       dr, int(window or 0), ctypes.c_float(scale), _p(out), _stream()))
 
 
+def wide_on_matrix_cores(dtype: torch.dtype, dk: int, dv: int) -> bool:
+    """Does `attend_heads` run on the matrix cores (bfloat16; keys in steps of 8, values in steps of 4, up to 256)?"""
+    return dtype == torch.bfloat16 and dk % 8 == 0 and 8 <= dk <= 256 and dv % 4 == 0 and 4 <= dv <= 256
+
+
 def attend_heads(ctx, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, pages: torch.Tensor, table: torch.Tensor,
-                 ring_pages: int, terms: "ScoreTerms", out: torch.Tensor) -> None:
-    """Attention of a step's rows over their own keys and values (k [n, H, dk], v [n, H, dv]) and, for cached positions,
-    those of `pages` (flat, of the kind that `KVGroup` keeps), nothing committed."""
-    H, dv = k.shape[1], v.shape[2]
-    attn_scored_plain(q, k, v, pages, H, dv, table, ring_pages, ctx.row_seq, ctx.row_pos, ctx.cu_seqlens, ctx.len_before,
-                      terms, None, out)
+                 ring_pages: int, window: Optional[int], scale: float, out: torch.Tensor) -> None:
+    """Attention of a step's rows over their own keys and values (k [n, H, dk], v [n, H, dv], a KV head for every query
+    head) and, for cached positions, those of `pages` (flat, of the kind that `KVGroup` keeps); nothing is committed.  On
+    the matrix cores where `wide_on_matrix_cores`, else in the plain kernel."""
+    n, H, dk = q.shape
+    dv = v.shape[2]
+    if not wide_on_matrix_cores(q.dtype, dk, dv):
+        attn_scored_plain(q, k, v, pages, H, dv, table, ring_pages, ctx.row_seq, ctx.row_pos, ctx.cu_seqlens, ctx.len_before,
+                          ScoreTerms(scale, window), None, out)
+        return
+    B = ctx.len_before.shape[0]
+    _req(q, "attend_heads.q", torch.bfloat16)
+    _req(k, "attend_heads.k", torch.bfloat16, (n, H, dk))
+    _req(v, "attend_heads.v", torch.bfloat16, (n, H, dv))
+    _req_pages(pages, H, dk, dv, "attend_heads")
+    stride = _req_table(table, B, "attend_heads")
+    _req(ctx.row_pos, "attend_heads.row_pos", torch.int32, (n,))
+    _req(ctx.cu_seqlens, "attend_heads.cu_seqlens", torch.int32, (B + 1,))
+    _req(ctx.tile_off, "attend_heads.tile_off", torch.int32, (B,))
+    _req(out, "attend_heads.out", torch.bfloat16, (n, H, dv))
+    vt = ctx.workspace.get("attend_heads_vt", (H, dv, ctx.host["aligned_cols"]), q.dtype)
+    v_tiles_rows(v, vt, ctx.cu_seqlens, ctx.tile_off, ctx.len_before, ctx.len_after)
+    n_tiles = int(sum(-(-int(x) // PREFILL_BLOCK) for x in ctx.host["n_new"]))
+    cuts = part = None
+    if not ctx.host.get("fixed_launches"):       # (a captured graph's launches must not be shaped by lengths)
+        at = ("prefill_cuts", window, H)
+        if at not in ctx.host:                   # the same for every layer of the step
+            ctx.host[at] = prefill_cuts(ctx.host["n_new"], ctx.host["len_before"], window, H, compute_units(q.device), q.device)
+        cuts = ctx.host[at]
+        if cuts is not None:
+            part = ctx.workspace.get("attn_prefill_part", (n * H * cuts.ways * (dv + 4),), torch.float32)
+    _check(lib().tl_attn_prefill_wide_bf16(_p(q), _p(k), _p(vt), vt.shape[2], _p(ctx.tile_off), _p(pages), _p(table), stride,
+                                           int(ring_pages), _p(ctx.row_pos), _p(ctx.cu_seqlens), _p(ctx.len_before), B,
+                                           cuts.n_items if cuts else n_tiles, H, H, dk, dv, int(window or 0),
+                                           ctypes.c_float(scale), _p(out), _p(cuts.items) if cuts else None,
+                                           _p(cuts.blocks) if cuts else None, cuts.n_cut if cuts else 0, _p(part),
+                                           cuts.ways if cuts else 0, ctypes.c_longlong(part.numel() if cuts else 0), n, _stream()))
 
 
 # ---- retention -----------------------------------------------------------------------------------------
@@ -1241,6 +1312,45 @@ def retention_norm_gate(o: torch.Tensor, gate: torch.Tensor, H: int, eps: float,
     _req(out, "retention_norm_gate.out", None, (n, inner))
     _check(lib().tl_retention_norm_gate(_p(o), _p(gate), gate.stride(0), n, H, inner // H, ctypes.c_float(eps), _p(out),
                                         _code(out.dtype), _stream()))
+
+
+def retention_chunk() -> int:
+    """Rows of a chunk of `retention_chunks`."""
+    return int(lib().tl_retention_chunk())
+
+
+def retention_chunks_serve(dtype: torch.dtype, dk: int, dv: int) -> bool:
+    """Does `retention_chunks` take this dtype and these heads?"""
+    return dtype == torch.bfloat16 and dk % 8 == 0 and 8 <= dk <= 256 and dv % 4 == 0 and 4 <= dv <= 256
+
+
+def retention_chunks(proj: torch.Tensor, row_pos, rotation, H: int, dk: int, dv: int, kscale: float, log2_decay: torch.Tensor,
+                     eps: float, state: torch.Tensor, cu_seqlens, slots, chunks: int, workspace, out: torch.Tensor) -> None:
+    """`retention_scan` and `retention_norm_gate` of a step with many rows, by chunks of `retention_chunk()` rows on the
+    matrix cores: proj float32 [n, 2 H (dk + dv)] = [q | k | v | g]; log2_decay float32 [H] (a decay of 0: a large negative
+    number); `chunks`: the sequences' new rows in chunks, every sequence's rounded up, added up; `workspace` gives the
+    scratch; out bfloat16 [n, H*dv]."""
+    n, width = proj.shape
+    B = slots.shape[0]
+    rot = _rotation(rotation, dk, "retention_chunks", magnitude=True)
+    _req(proj, "retention_chunks.proj", torch.float32, (n, 2 * H * (dk + dv)))
+    _req(row_pos, "retention_chunks.row_pos", torch.int32, (n,))
+    _req(log2_decay, "retention_chunks.log2_decay", torch.float32, (H,))
+    _req_state(state, H * dk * dv, "retention_chunks")
+    _req(cu_seqlens, "retention_chunks.cu_seqlens", torch.int32, (B + 1,))
+    _req(slots, "retention_chunks.slots", torch.int32)
+    _req(out, "retention_chunks.out", torch.bfloat16, (n, H * dv))
+    if not retention_chunks_serve(out.dtype, dk, dv):
+        raise KernelError(f"retention_chunks: heads of {dk} and {dv} are not served")
+    C, bf, get = retention_chunk(), torch.bfloat16, workspace.get
+    scratch = (get("retc_q", (n * H * dk,), bf), get("retc_k", (n * H * dk,), bf), get("retc_kt_hi", (chunks * H * dk * C,), bf),
+               get("retc_kt_lo", (chunks * H * dk * C,), bf), get("retc_vt", (chunks * H * dv * C,), bf),
+               get("retc_kv", (chunks * H * dk * dv,), torch.float32), get("retc_st_hi", (chunks * H * dk * dv,), bf),
+               get("retc_st_lo", (chunks * H * dk * dv,), bf))
+    _check(lib().tl_retention_chunks(_p(proj), width, H, dk, dv, _p(row_pos), _p(rot.inv_freq), rot.rotary_dim,
+                                     int(rot.interleaved), ctypes.c_float(rot.magnitude), ctypes.c_float(kscale), _p(log2_decay),
+                                     ctypes.c_float(eps), _p(state), ctypes.c_longlong(state.stride(0)), _p(cu_seqlens), _p(slots), n,
+                                     B, int(chunks), *[_p(t) for t in scratch], _p(out), _stream()))
 
 
 def take_tokens(src: torch.Tensor, idx: torch.Tensor, vocab: int, tokens: torch.Tensor) -> None:

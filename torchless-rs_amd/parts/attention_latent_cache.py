@@ -107,7 +107,6 @@ class LatentCacheAttentionMixer(Mixer):
         uk = t("uk").to(compute_dtype).view(self.nq, self.dn, self.R)
         self.uk_t = uk.transpose(1, 2).contiguous()
         self.uv = t("uv").to(compute_dtype).view(self.nq, self.dv, self.R).contiguous()
-        self.terms = ops.ScoreTerms(self.scale, self.window)
 
     # ---- one step --------------------------------------------------------------
     def produce(self, ctx, run, y: torch.Tensor, out: torch.Tensor):
@@ -150,7 +149,7 @@ class LatentCacheAttentionMixer(Mixer):
             v = ws.get("latc_v", (n, nq, dv), ctx.dtype)
             ops.latent_heads(kvf, rows[:, R:], nq, dn, dr, dv, k, v)
             old, old_table = self._cached_heads(ctx, group, run.kv_group_index, pages, table)
-            ops.attend_heads(ctx, q, k, v, old, old_table, group.ring_pages, self.terms, att)
+            ops.attend_heads(ctx, q, k, v, old, old_table, group.ring_pages, self.window, self.scale, att)
             ops.latent_commit(rows, ctx.row_seq, ctx.row_pos, ctx.len_after, table, group.ring_pages, pages)
         self.o(att.view(n, nq * dv), out)
         return None

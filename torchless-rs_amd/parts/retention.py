@@ -17,6 +17,7 @@ Single tokens, short portions and the 32-bit path go row by row with everything 
 """
 from __future__ import annotations
 
+import math
 from typing import Dict, Optional, Sequence
 
 import torch
@@ -26,6 +27,9 @@ from ..kernels import ops
 from ..weights.binding import WeightSpec
 from .base import Mixer, PartSpec, make_part, register_part
 from .linear import Linear
+
+CHUNKS_FROM = 32             # a bfloat16 step whose longest sequence brings this many rows goes by chunks
+NO_DECAY_LEFT = -10000.0     # log2 of a decay of 0, as the chunks' kernels take it
 
 
 class RetentionMixer(Mixer):
@@ -72,6 +76,8 @@ class RetentionMixer(Mixer):
         self.proj = Linear(torch.cat(ws, dim=0), tiled=True)
         self.o = Linear(tensors[p + nm["o"]], tiled=True)
         self.decay = torch.tensor(self.decay_host, dtype=torch.float64).to(torch.float32).to(ws[0].device)
+        logs = [math.log2(a) if a > 0.0 else NO_DECAY_LEFT for a in self.decay_host]
+        self.log2_decay = torch.tensor(logs, dtype=torch.float64).to(torch.float32).to(ws[0].device)
 
     def _heads(self, ctx, run, y: torch.Tensor) -> torch.Tensor:
         """The normed and gated heads [n, H * dv] in the compute dtype."""
@@ -81,6 +87,12 @@ class RetentionMixer(Mixer):
         self.proj(y, proj)
         rotation = self.position.rotation(y.device) or ops.NO_ROTATION
         h = ws.get("ret_h", (n, H * dv), ctx.dtype)
+        if ctx.max_new >= CHUNKS_FROM and ops.retention_chunks_serve(ctx.dtype, dk, dv):
+            C = ops.retention_chunk()
+            chunks = int(sum(-(-int(r) // C) for r in ctx.host["n_new"]))
+            ops.retention_chunks(proj, ctx.row_pos, rotation, H, dk, dv, self.kscale, self.log2_decay, self.eps, run.state,
+                                 ctx.cu_seqlens, ctx.slots, chunks, ws, h)
+            return h
         o = ws.get("ret_o", (n, H * dv), torch.float32)
         ops.retention_scan(proj, ctx.row_pos, rotation, H, dk, dv, self.kscale, self.decay, run.state, ctx.cu_seqlens,
                            ctx.slots, o)
