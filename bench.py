@@ -236,9 +236,73 @@ def giforax_counts(z: dict, layers: int, B: int, C: int, T: int):
     return w, kv, att, w_read
 
 
+def zudalorn_layers(layers: int):
+    """(mixer, feed-forward) of `zudalorn_config(z, layers)`: both mixers with both feed-forwards in every four layers."""
+    kinds = [("retention", "dense"), ("latent_attention", "moe"), ("retention", "moe"), ("latent_attention", "dense")]
+    return [kinds[i % 4] for i in range(layers)]
+
+
+def zudalorn_sizes(z: dict):
+    """Sizes of the Zudalorn layers at the layer sizes `z`: as many heads of the same size in both mixers, latents of four
+    heads' channels with half a head rotated beside them; an ungated feed-forward half as wide again as the gated one; 16
+    gated experts of an eighth of its hidden size of which a token uses 4, beside a shared one of half of it: a token
+    multiplies as much as in the dense gated feed-forward either way."""
+    return dict(rank=4 * z["dim"], rot=z["dim"] // 2, dense_ff=3 * z["ff"] // 2, experts=16, top=4, expert_ff=z["ff"] // 8,
+                shared_ff=z["ff"] // 2)
+
+
+def zudalorn_config(z: dict, layers: int):
+    """config.json of a Zudalorn model with the layer sizes `z` (see `zudalorn_layers`, `zudalorn_sizes`)."""
+    n = zudalorn_sizes(z)
+    out = []
+    for mix, ff in zudalorn_layers(layers):
+        if mix == "retention":
+            m = {"heads": z["heads"], "dim": z["dim"], "vdim": z["dim"], "rot": {"base": 10000.0, "dims": z["dim"]},
+                 "decay": [1.0 - 2.0 ** (-5.0 - 7.0 * h / max(1, z["heads"] - 1)) for h in range(z["heads"])]}
+        else:
+            m = {"heads": z["heads"], "dim": z["dim"], "rot_dim": n["rot"], "vdim": z["dim"], "kv_rank": n["rank"],
+                 "scale": (z["dim"] + n["rot"]) ** -0.5,
+                 "rot": {"base": 10000.0, "dims": n["rot"], "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+            if z["window"]:
+                m["mask"] = {"size": z["window"]}
+        mlp = {"kind": "dense", "ff": n["dense_ff"]} if ff == "dense" else {
+            "kind": "moe", "router": {"experts": n["experts"], "top": n["top"], "groups": {"count": 4, "keep": 2}},
+            "expert": {"ff": n["expert_ff"]}, "shared": {"ff": n["shared_ff"]}}
+        out.append({"type": mix, "mixer": m, "mlp": mlp})
+    return {"architecture": "Zudalorn", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6}, "layers": out}
+
+
+def zudalorn_counts(z: dict, layers: int, B: int, C: int, T: int):
+    """(weight elements that a prompt's products multiply a row by, bytes of cached latents and recurrent state that a
+    decode step reads and writes, multiply-adds times two of a prompt's attention and recurrence, weight elements that
+    a decode step of B rows must read) of `zudalorn_config(z, layers)`.  A prompt makes keys and values per head of its
+    latents; a decode step reads the latents as they are."""
+    H, nq, d = z["width"], z["heads"], z["dim"]
+    n = zudalorn_sizes(z)
+    w = w_read = kv = att = 0
+    for mix, ff in zudalorn_layers(layers):
+        if mix == "retention":
+            m = 5 * nq * d * H
+            kv += B * nq * d * d * 4 * 2
+            att += 4 * T * nq * d * d
+        else:
+            m = nq * (d + n["rot"]) * H + (n["rank"] + n["rot"]) * H + 2 * nq * d * n["rank"] + nq * d * H
+            kv += B * (min(C, z["window"]) if z["window"] else C) * (n["rank"] + n["rot"]) * 2
+            att += 2 * nq * (2 * d + n["rot"]) * sum(min(p + 1, z["window"] or T) for p in range(T))
+        w += m
+        w_read += m
+        if ff == "dense":
+            w += 2 * H * n["dense_ff"]
+            w_read += 2 * H * n["dense_ff"]
+        else:
+            w += 3 * H * (n["top"] * n["expert_ff"] + n["shared_ff"]) + n["experts"] * H
+            w_read += 3 * H * (min(n["experts"], B * n["top"]) * n["expert_ff"] + n["shared_ff"]) + n["experts"] * H
+    return w, kv, att, w_read
+
+
 def bench_designs(args) -> int:
     """Prefill (one prompt of --prefill-tokens in one step) and decode (--batch sequences at --context
-    positions, one token a step through captured graphs) of the three designs at equal layer sizes,
+    positions, one token a step through captured graphs) of the designs at equal layer sizes,
     random weights, bfloat16.  The bytes a decode step must read (every weight once, the live keys
     and values) over its time is its share of the HBM roofline; a prefill's products and causal
     attention over its time its share of the matrix cores' peak."""
@@ -321,6 +385,8 @@ def bench_designs(args) -> int:
             row["nepisun"] = measure(nepisun_config(z, L), z, counts=nepisun_counts(z, L, B, C, T))
         if "giforax" in which:
             row["giforax"] = measure(giforax_config(z, L), z, counts=giforax_counts(z, L, B, C, T))
+        if "zudalorn" in which:
+            row["zudalorn"] = measure(zudalorn_config(z, L), z, counts=zudalorn_counts(z, L, B, C, T))
         if "sozetar" in which:
             row["sozetar"] = measure(soz, z)
         if "mistral" in which:
@@ -355,10 +421,10 @@ def main() -> int:
     ap.add_argument("--only", choices=["prefill", "decode", "pipes", "designs"], default=None,
                     help="measure one phase only and print its line to stderr (for profiling); pipes: whether a "
                          "SIMD's matrix and vector pipes overlap (ops.measure_pipes); designs: prefill and decode of "
-                         "the Fanitar, Sozetar, Nepisun and Giforax designs beside the Mistral design at equal layer sizes (--design-sizes, "
+                         "the Fanitar, Sozetar, Nepisun, Giforax and Zudalorn designs beside the Mistral design at equal layer sizes (--design-sizes, "
                          "--layers, --batch, --context, --prefill-tokens apply)")
     ap.add_argument("--design-names", default="fanitar,sozetar,mistral",
-                    help="with --only designs: which designs to run (of fanitar, sozetar, nepisun, giforax, mistral)")
+                    help="with --only designs: which designs to run (of fanitar, sozetar, nepisun, giforax, zudalorn, mistral)")
     ap.add_argument("--design-sizes", default="2b,7b,12b",
                     help="with --only designs: which layer sizes to run (of %s)" % ",".join(sorted(DESIGN_SIZES)))
     args = ap.parse_args()

@@ -160,6 +160,35 @@ expert_act_kernel(const float* __restrict__ u, const float* __restrict__ weights
   }
 }
 
+// out[i] = act(u[i]) over `total` elements (a multiple of 8), u float or bfloat16: the activation of a plain feed-forward
+template <typename U, typename T>
+__global__ void __launch_bounds__(256)
+unary_act_kernel(const U* __restrict__ u, size_t total, UnaryAct act, T* __restrict__ out) {
+  for (size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * 8; i < total; i += (size_t)gridDim.x * 256 * 8) {
+    float z[8];
+    if constexpr (sizeof(U) == 2) {
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>(u + i);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) z[e] = (float)v[e];
+    } else {
+      const f32x4 a = *reinterpret_cast<const f32x4*>(u + i), b = *reinterpret_cast<const f32x4*>(u + i + 4);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        z[e] = a[e];
+        z[4 + e] = b[e];
+      }
+    }
+    if constexpr (sizeof(T) == 2) {
+      bf16x8 r;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) r[e] = (bf16)unary_act(z[e], act);
+      *reinterpret_cast<bf16x8*>(out + i) = r;
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) out[i + e] = unary_act(z[e], act);
+    }
+  }
+}
 
 // ---- the chosen experts alone, row by row ---------------------------------------------------------------
 // For steps of few rows (fewer chosen experts than there are experts) the wide feed-forward would read every
@@ -382,6 +411,22 @@ int tl_expert_act(const float* u, const float* weights, const float* shared_w, i
   else
     TL_REQUIRE(false, "expert_act: unknown dtype code %d", dt);
   TL_LAUNCH_CHECK("expert_act");
+  return 0;
+}
+
+// u (dtype udt) and out (dtype dt) of `total` elements, a multiple of 8, 16-byte aligned
+int tl_unary_act(const void* u, int udt, long long total, int act_code, float act_a, float act_b, void* out, int dt, hipStream_t st) {
+  const UnaryAct act{act_code, act_a, act_b};
+  TL_REQUIRE(total >= 0 && total % 8 == 0 && act_code >= 0 && act_code <= 2, "unary_act: bad sizes total=%lld act=%d", total, act_code);
+  TL_REQUIRE(u && out && (uintptr_t)u % 16 == 0 && (uintptr_t)out % 16 == 0, "unary_act: a buffer is missing or off 16 bytes");
+  if (total == 0) return 0;
+  const long long want = (total / 8 + 255) / 256;
+  const unsigned blocks = (unsigned)(want < 8192 ? want : 8192);
+  if (udt == DT_F32 && dt == DT_F32) unary_act_kernel<float, float><<<blocks, 256, 0, st>>>((const float*)u, (size_t)total, act, (float*)out);
+  else if (udt == DT_F32 && dt == DT_BF16) unary_act_kernel<float, bf16><<<blocks, 256, 0, st>>>((const float*)u, (size_t)total, act, (bf16*)out);
+  else if (udt == DT_BF16 && dt == DT_BF16) unary_act_kernel<bf16, bf16><<<blocks, 256, 0, st>>>((const bf16*)u, (size_t)total, act, (bf16*)out);
+  else TL_REQUIRE(false, "unary_act: unknown dtype codes %d and %d", udt, dt);
+  TL_LAUNCH_CHECK("unary_act");
   return 0;
 }
 

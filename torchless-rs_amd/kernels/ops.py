@@ -1028,6 +1028,14 @@ def expert_act(u: torch.Tensor, weights: Optional[torch.Tensor], E: int, ff: int
                                _p(out), _code(out.dtype), _stream()))
 
 
+def unary_act(u: torch.Tensor, activation: str, out: torch.Tensor, constants=None) -> None:
+    """out = act(u) element by element (u float32, or bfloat16 like out; any number of elements that is a multiple of 8)."""
+    code = _unary_args(activation, constants)
+    _req(u, "unary_act.u", u.dtype if u.dtype == torch.float32 else out.dtype)
+    _req(out, "unary_act.out", None, u.shape)
+    _check(lib().tl_unary_act(_p(u), _code(u.dtype), ctypes.c_longlong(u.numel()), *code, _p(out), _code(out.dtype), _stream()))
+
+
 def expert_rows_up(y: torch.Tensor, up: torch.Tensor, chosen: torch.Tensor, weights: torch.Tensor, ff: int, shared: int,
                    activation: str, hs: torch.Tensor, constants=None, shared_weight: Optional[torch.Tensor] = None) -> None:
     """The chosen experts' first halves, row by row: hs[n, k*ff + j] = act(up[chosen[n,k]*ff + j] . y[n]) * weights[n, chosen[n,k]]
@@ -1189,23 +1197,19 @@ def latents_on_matrix_cores(dtype: torch.dtype, R: int, dr: int) -> bool:
 
 
 @functools.lru_cache(maxsize=4096)
-def latent_splits(B: int, H: int, R: int, max_pages: int, units: int):
-    """(head groups of 16 that a workgroup takes, splits of the pages): a workgroup stages a page once for all its heads, so
-    the more heads the fewer bytes, unless compute units stand idle for it; splits as `decode_splits` weighs them."""
-    groups = -(-H // 16)
-    per_unit = 1 if R > 256 else 2                    # a page's rows fill half of a compute unit's LDS, or more
-    room = units * per_unit
-    best = None
-    for hg in (1, 2, 4):
-        if hg > 1 and hg >= 2 * groups:
-            break
-        wide = B * -(-groups // hg)
-        step = 1.0 + 0.25 * (hg - 1)                  # what a page costs with more heads on it
-        for s in range(1, max_pages + 1):
-            cost = -(-wide * s // room) * -(-max_pages // s) * step + SPLIT_COST * s
-            if best is None or cost < best[0] - 1e-9:
-                best = (cost, hg, s)
-    return best[1], best[2]
+def latent_splits(B: int, H: int, R: int, D: int, max_pages: int, units: int) -> int:
+    """Into how many parts the cached rows of a single-token step are cut, by what was measured (us): 4 to start, 4 for a page
+    of 576 channels in a workgroup that has a compute unit to itself and 5 where two share it, and the parts' sums written
+    and read back at 2 TB/s."""
+    wide = B * -(-H // 16)
+
+    def cost(s):
+        rounds = -(-wide * s // (2 * units))
+        page = (4.0 if wide * s <= units else 5.0) * max(D, 128) / 576.0
+        return 4.0 + rounds * -(-max_pages // s) * page + (2.0 + B * H * s * R * 8 / 2e6 if s > 1 else 0.0)
+
+    most = max(1, min(max_pages, 4 * units // wide + 1, 1024))
+    return min(range(1, most + 1), key=lambda s: (cost(s), s))
 
 
 def latent_attention(q: torch.Tensor, pages: torch.Tensor, table: torch.Tensor, ring_pages: int, ctx, dr: int,
@@ -1221,10 +1225,10 @@ def latent_attention(q: torch.Tensor, pages: torch.Tensor, table: torch.Tensor, 
     _req(out, "latent_attention.out", q.dtype, (B, H, R))
     if latents_on_matrix_cores(q.dtype, R, dr):
         most = stride if not window else min(stride, -(-window // PAGE) + 1)
-        hg, splits = latent_splits(B, H, R, min(most, 4096), compute_units(q.device))     # (by the table's width: fixed while a graph lives)
+        splits = latent_splits(B, H, R, D, most, compute_units(q.device))      # by the table's width: fixed while a graph lives
         part = ctx.workspace.get("latent_part", (B * H * splits * (R + 2),), torch.float32) if splits > 1 else None
         _check(lib().tl_latent_decode_bf16(_p(q), _p(pages), _p(table), stride, int(ring_pages), _p(ctx.row_pos), B, H, R, dr,
-                                           int(window or 0), ctypes.c_float(scale), hg, splits, _p(part), _p(out), _stream()))
+                                           int(window or 0), ctypes.c_float(scale), splits, _p(part), _p(out), _stream()))
         return
     _check(lib().tl_latent_attn_plain(_p(q), _p(pages), _code(q.dtype), _p(table), stride, int(ring_pages), _p(ctx.row_pos), B, H, R,
                                       dr, int(window or 0), ctypes.c_float(scale), _p(out), _stream()))
@@ -1242,7 +1246,7 @@ def attend_heads(ctx, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, pages: 
     the matrix cores where `wide_on_matrix_cores`, else in the plain kernel."""
     n, H, dk = q.shape
     dv = v.shape[2]
-    if not wide_on_matrix_cores(q.dtype, dk, dv):
+    if not wide_on_matrix_cores(q.dtype, dk, dv) or not scale > 0.0:
         attn_scored_plain(q, k, v, pages, H, dv, table, ring_pages, ctx.row_seq, ctx.row_pos, ctx.cu_seqlens, ctx.len_before,
                           ScoreTerms(scale, window), None, out)
         return

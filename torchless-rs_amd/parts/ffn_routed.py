@@ -91,10 +91,17 @@ class PlainFeedForward(FeedForward):
 
     def _hidden(self, ctx, y: torch.Tensor) -> torch.Tensor:
         n = y.shape[0]
-        u = ctx.workspace.get("pff_u", (n, self.I), torch.float32)
-        self.up(y, u)
         h = ctx.workspace.get("pff_h", (n, self.I), ctx.dtype)
-        ops.expert_act(u, None, 0, self.I, self.activation, h, self.constants)
+        if not self.up.own_kernels(n) and self.I % 8 == 0 and ops.bf16_gemm_ok(y, self.up.weight):
+            u = ctx.workspace.get("pff_u16", (n, self.I), torch.bfloat16)      # many rows: half the traffic, one rounding more
+            ops.gemm_library(y, self.up.weight, u)
+        else:
+            u = ctx.workspace.get("pff_u", (n, self.I), torch.float32)
+            self.up(y, u)
+        if self.I % 8 == 0:
+            ops.unary_act(u, self.activation, h, self.constants)
+        else:
+            ops.expert_act(u, None, 0, self.I, self.activation, h, self.constants)
         return h
 
     def forward(self, ctx, y: torch.Tensor, x: torch.Tensor) -> None:
