@@ -488,11 +488,13 @@ def test_single_tokens_over_cached_latents(dtype, H, R, dr, window):
 
 
 @pytest.mark.parametrize("splits", [1, 2, 3, 9, 40])
-def test_splits_of_the_cached_latents(splits, monkeypatch):
-    """A loud row in the first page, one in the last, and long runs without; more splits than pages leave some empty."""
+@pytest.mark.parametrize("blocks, H, R, dr", [(1, 6, 128, 16), (1, 16, 510, 66), (1, 33, 504, 8), (2, 6, 512, 64), (2, 48, 510, 66)])
+def test_splits_of_the_cached_latents(splits, blocks, H, R, dr, monkeypatch):
+    """A loud row in the first page, one in the last, and long runs without; more splits than pages leave some empty.
+    One and two blocks of 16 heads a workgroup."""
     from torchless_rs_amd.kernels import ops
-    monkeypatch.setattr(ops, "latent_splits", lambda *a: splits)
-    H, R, dr, L = 6, 128, 16, 1000
+    monkeypatch.setattr(ops, "latent_splits", lambda *a: (blocks, splits))
+    L = 1000
     D, n = R + dr, 16
     rows, q = loud_rows(L, D, H, [3, L - 2], seed=1)
     rows, q = rows.bfloat16(), q.bfloat16()

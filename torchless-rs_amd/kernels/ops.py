@@ -1197,19 +1197,23 @@ def latents_on_matrix_cores(dtype: torch.dtype, R: int, dr: int) -> bool:
 
 
 @functools.lru_cache(maxsize=4096)
-def latent_splits(B: int, H: int, R: int, D: int, max_pages: int, units: int) -> int:
-    """Into how many parts the cached rows of a single-token step are cut, by what was measured (us): 4 to start, 4 for a page
-    of 576 channels in a workgroup that has a compute unit to itself and 5 where two share it, and the parts' sums written
-    and read back at 2 TB/s."""
-    wide = B * -(-H // 16)
+def latent_splits(B: int, H: int, R: int, D: int, max_pages: int, units: int):
+    """(blocks of 16 heads a workgroup, parts that the cached rows are cut into) of a single-token step, by what was
+    measured (us, rows of 576 channels): 8 to start and 2.2 a page for a workgroup of one block that has a compute unit to
+    itself, 4 where two share it; 11 to start and 3.3 a page with two blocks; the parts' sums 3 and what they take to be
+    written and read back at 3 TB/s."""
+    def cost(blocks, s):
+        groups = B * -(-H // (16 * blocks)) * s
+        if blocks == 2:
+            start, page, at_once = 11.0, 3.3, units
+        else:
+            start, page, at_once = 8.0, 2.2 if groups <= units else 4.0, 2 * units
+        return (start + -(-groups // at_once) * -(-max_pages // s) * page * max(D, 128) / 576.0
+                + (3.0 + B * H * s * R * 8 / 3e6 if s > 1 else 0.0))
 
-    def cost(s):
-        rounds = -(-wide * s // (2 * units))
-        page = (4.0 if wide * s <= units else 5.0) * max(D, 128) / 576.0
-        return 4.0 + rounds * -(-max_pages // s) * page + (2.0 + B * H * s * R * 8 / 2e6 if s > 1 else 0.0)
-
-    most = max(1, min(max_pages, 4 * units // wide + 1, 1024))
-    return min(range(1, most + 1), key=lambda s: (cost(s), s))
+    most = max(1, min(max_pages, 4 * units // (B * -(-H // 16)) + 1, 1024))
+    kinds = (1, 2) if R > 256 and D == 576 and H > 16 else (1,)
+    return min(((k, s) for s in range(1, most + 1) for k in kinds), key=lambda ks: (cost(*ks), ks[1]))
 
 
 def latent_attention(q: torch.Tensor, pages: torch.Tensor, table: torch.Tensor, ring_pages: int, ctx, dr: int,
@@ -1225,10 +1229,11 @@ def latent_attention(q: torch.Tensor, pages: torch.Tensor, table: torch.Tensor, 
     _req(out, "latent_attention.out", q.dtype, (B, H, R))
     if latents_on_matrix_cores(q.dtype, R, dr):
         most = stride if not window else min(stride, -(-window // PAGE) + 1)
-        splits = latent_splits(B, H, R, D, most, compute_units(q.device))      # by the table's width: fixed while a graph lives
-        part = ctx.workspace.get("latent_part", (B * H * splits * (R + 2),), torch.float32) if splits > 1 else None
+        blocks, splits = latent_splits(B, H, R, D, most, compute_units(q.device))      # by the table's width: fixed while a graph lives
+        line = int(lib().tl_latent_part_line(R))
+        part = ctx.workspace.get("latent_part", (B * H * splits * line,), torch.float32) if splits > 1 else None
         _check(lib().tl_latent_decode_bf16(_p(q), _p(pages), _p(table), stride, int(ring_pages), _p(ctx.row_pos), B, H, R, dr,
-                                           int(window or 0), ctypes.c_float(scale), splits, _p(part), _p(out), _stream()))
+                                           int(window or 0), ctypes.c_float(scale), splits, blocks, _p(part), _p(out), _stream()))
         return
     _check(lib().tl_latent_attn_plain(_p(q), _p(pages), _code(q.dtype), _p(table), stride, int(ring_pages), _p(ctx.row_pos), B, H, R,
                                       dr, int(window or 0), ctypes.c_float(scale), _p(out), _stream()))
