@@ -2,7 +2,7 @@
 //
 // A row of the projection is [q (nq*dk) | k (nkv*dk) | v (nkv*dv) | g (ng)] in float.  Per row:
 //
-//   * the biases are added (optional);
+//   * the biases are added (optional), and the values multiplied by `v_factor`;
 //   * every head of q and of k is divided by ITS OWN root mean square over its dk channels,
 //     eps inside the root, and multiplied by a weight of dk channels that all heads share
 //     (optional; q and k have a weight each);
@@ -35,11 +35,12 @@ struct HeadTerms {
   float lambda;
   float* v_first;          // [n, nkv*dv] float
   int unit_norm;           // q and k heads divided by their root mean square after the rotation, no weight
+  float v_factor;          // on the (biased) values
 };
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-head_prepare_kernel(const float* __restrict__ proj, const int* __restrict__ row_pos, Rotation rot, HeadTerms t,
+head_prepare_kernel(const float* __restrict__ proj, int proj_stride, const int* __restrict__ row_pos, Rotation rot, HeadTerms t,
                     int nq, int nkv, int dk, int dv, int ng, T* __restrict__ q, T* __restrict__ k, T* __restrict__ v,
                     float* __restrict__ gate, const int* __restrict__ table, int table_stride, int ring_pages,
                     T* __restrict__ pages) {
@@ -49,7 +50,7 @@ head_prepare_kernel(const float* __restrict__ proj, const int* __restrict__ row_
   const int Q = nq * dk, K = nkv * dk, V = nkv * dv;
   const int gate_units = (ng + 255) / 256;
   if (unit >= nq + 2 * nkv + gate_units) return;
-  const float* row = proj + (size_t)n * (Q + K + V + ng);
+  const float* row = proj + (size_t)n * proj_stride;
   const int pos = row_pos[n];
   auto at = [&](int i) { return row[i] + (t.bias ? t.bias[i] : 0.f); };
 
@@ -114,7 +115,7 @@ head_prepare_kernel(const float* __restrict__ proj, const int* __restrict__ row_
     const int head = unit - nq - nkv;
     for (int c = lane; c < dv; c += WAVE) {
       const int i = head * dv + c;
-      float a = at(Q + K + i);
+      float a = at(Q + K + i) * t.v_factor;
       if (t.mix == 1) t.v_first[(size_t)n * V + i] = a;
       else if (t.mix == 2) a = (1.0f - t.lambda) * a + t.lambda * t.v_first[(size_t)n * V + i];
       const T o = from_f32<T>(a);
@@ -134,12 +135,13 @@ using namespace tl;
 
 extern "C" {
 
-int tl_head_prepare(const float* proj, const int* row_pos, const float* inv_freq, int rotary_dim, const float* bias,
-                    const float* q_norm, const float* k_norm, float eps, int unit_norm, int mix, float lambda, float* v_first,
-                    int n, int nq, int nkv, int dk, int dv, int ng, void* q, void* k, void* v, float* gate, int dt,
+int tl_head_prepare(const float* proj, int proj_stride, const int* row_pos, const float* inv_freq, int rotary_dim, const float* bias,
+                    const float* q_norm, const float* k_norm, float eps, int unit_norm, int mix, float lambda, float v_factor,
+                    float* v_first, int n, int nq, int nkv, int dk, int dv, int ng, void* q, void* k, void* v, float* gate, int dt,
                     const int* table, int table_stride, int ring_pages, void* pages, hipStream_t st) {
   TL_REQUIRE(n >= 0 && nq > 0 && nkv >= 0 && dk > 0 && dv > 0 && ng >= 0 && dk <= HP_MAX_D && dv <= HP_MAX_D,
              "head_prepare: bad sizes n=%d nq=%d nkv=%d dk=%d dv=%d ng=%d (heads up to %d)", n, nq, nkv, dk, dv, ng, HP_MAX_D);
+  TL_REQUIRE(proj_stride >= nq * dk + nkv * (dk + dv) + ng, "head_prepare: rows %d apart are too short", proj_stride);
   TL_REQUIRE(rotary_dim >= 0 && rotary_dim % 2 == 0 && rotary_dim <= dk,
              "head_prepare: %d rotated channels of a head of %d (even, at most the head)", rotary_dim, dk);
   TL_REQUIRE(rotary_dim == 0 || inv_freq, "head_prepare: a rotation without frequencies");
@@ -151,14 +153,14 @@ int tl_head_prepare(const float* proj, const int* row_pos, const float* inv_freq
   TL_REQUIRE(dt == DT_F32 || dt == DT_BF16, "head_prepare: unknown dtype code %d", dt);
   if (n == 0) return 0;
   const Rotation rot{inv_freq, rotary_dim, 0};
-  const HeadTerms t{bias, q_norm, k_norm, eps, mix, lambda, v_first, unit_norm};
+  const HeadTerms t{bias, q_norm, k_norm, eps, mix, lambda, v_first, unit_norm, v_factor};
   const int units = nq + 2 * nkv + (ng + 255) / 256;
   const dim3 grid(n, (units + 3) / 4);
   if (dt == DT_F32)
-    head_prepare_kernel<float><<<grid, 256, 0, st>>>(proj, row_pos, rot, t, nq, nkv, dk, dv, ng, (float*)q, (float*)k,
+    head_prepare_kernel<float><<<grid, 256, 0, st>>>(proj, proj_stride, row_pos, rot, t, nq, nkv, dk, dv, ng, (float*)q, (float*)k,
                                                      (float*)v, gate, table, table_stride, ring_pages, (float*)pages);
   else
-    head_prepare_kernel<bf16><<<grid, 256, 0, st>>>(proj, row_pos, rot, t, nq, nkv, dk, dv, ng, (bf16*)q, (bf16*)k,
+    head_prepare_kernel<bf16><<<grid, 256, 0, st>>>(proj, proj_stride, row_pos, rot, t, nq, nkv, dk, dv, ng, (bf16*)q, (bf16*)k,
                                                     (bf16*)v, gate, table, table_stride, ring_pages, (bf16*)pages);
   TL_LAUNCH_CHECK("head_prepare");
   return 0;

@@ -25,6 +25,55 @@ __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict_
   for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = to_f32(row[i]) * scale;
 }
 
+// The same with a second table read by pairs of tokens, and a norm of the sum: row (previous * mul_prev + current * mul_cur)
+// mod buckets of `pairs`, row `buckets` for a sequence's first token.  The previous token of a sequence's first row of the
+// step lies in `last`; the workgroup of that row alone reads and then replaces it.  One workgroup a row; the row's sum goes
+// through `out` (every thread reads back what it wrote).
+struct PairTerms {
+  const int* row_pos;
+  const int* row_seq;
+  const int* cu_seqlens;
+  const int* slots;
+  int* last;
+  long long buckets, mul_prev, mul_cur;
+};
+template <typename T>
+__global__ void __launch_bounds__(256)
+embed_pairs_kernel(const T* __restrict__ table, const int* __restrict__ ids, int H, float scale, const T* __restrict__ pairs, PairTerms k,
+                   const float* __restrict__ w, float eps, float* __restrict__ out) {
+  __shared__ float sh[4];
+  __shared__ int s_prev;
+  const int n = blockIdx.x;
+  const T* row = table + (size_t)ids[n] * H;
+  const T* second = nullptr;
+  if (pairs) {
+    const int b = k.row_seq[n], row0 = k.cu_seqlens[b];
+    if (threadIdx.x == 0) {
+      int prev = n > row0 ? ids[n - 1] : k.last[k.slots[b]];
+      if (k.row_pos[n] == 0) prev = -1;
+      s_prev = prev;
+      if (n == row0) k.last[k.slots[b]] = ids[k.cu_seqlens[b + 1] - 1];
+    }
+    __syncthreads();
+    const int prev = s_prev;
+    // (two products of 31 bits each fit 63)
+    const long long at = prev < 0 ? k.buckets : (prev * k.mul_prev + ids[n] * k.mul_cur) % k.buckets;
+    second = pairs + (size_t)at * H;
+  }
+  float* o = out + (size_t)n * H;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < H; i += 256) {
+    float a = to_f32(row[i]) * scale;
+    if (second) a += to_f32(second[i]);
+    o[i] = a;
+    ss += a * a;
+  }
+  if (w == nullptr) return;
+  ss = block_sum<256>(ss, sh);
+  const float rms = sqrtf(ss / (float)H + eps);
+  for (int i = threadIdx.x; i < H; i += 256) o[i] = (o[i] / rms) * w[i];
+}
+
 // ---- RMSNorm: y = x / sqrt(mean(x^2) + eps) * w ------------------------------
 // src/kernels/mod.rs:558-568 of the reference: eps inside the root, divide,
 // then multiply by the weight.
@@ -735,6 +784,24 @@ int tl_embed(const void* table, int table_dt, const int* ids, int n, int H, floa
   else
     TL_REQUIRE(false, "embed: unknown dtype code %d", table_dt);
   TL_LAUNCH_CHECK("embed");
+  return 0;
+}
+
+int tl_embed_pairs(const void* table, int table_dt, const int* ids, int n, int H, float scale, const void* pairs, long long buckets,
+                   long long mul_prev, long long mul_cur, const int* row_pos, const int* row_seq, const int* cu_seqlens,
+                   const int* slots, int* last, const float* w, float eps, float* out, hipStream_t st) {
+  TL_REQUIRE(n >= 0 && H > 0 && table && ids && out, "embed_pairs: bad arguments n=%d H=%d", n, H);
+  TL_REQUIRE(!pairs || (row_pos && row_seq && cu_seqlens && slots && last), "embed_pairs: a buffer is missing");
+  TL_REQUIRE(buckets > 0 && mul_prev >= 0 && mul_cur >= 0 && mul_prev < (1LL << 31) && mul_cur < (1LL << 31),
+             "embed_pairs: multipliers must lie between 0 and 2^31, buckets above 0");
+  TL_REQUIRE(table_dt == DT_F32 || table_dt == DT_BF16, "embed_pairs: unknown dtype code %d", table_dt);
+  if (n == 0) return 0;
+  const PairTerms k{row_pos, row_seq, cu_seqlens, slots, last, buckets, mul_prev, mul_cur};
+  if (table_dt == DT_F32)
+    embed_pairs_kernel<float><<<n, 256, 0, st>>>((const float*)table, ids, H, scale, (const float*)pairs, k, w, eps, out);
+  else
+    embed_pairs_kernel<bf16><<<n, 256, 0, st>>>((const bf16*)table, ids, H, scale, (const bf16*)pairs, k, w, eps, out);
+  TL_LAUNCH_CHECK("embed_pairs");
   return 0;
 }
 

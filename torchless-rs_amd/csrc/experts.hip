@@ -1,6 +1,6 @@
 // A routed mixture of small feed-forward layers ("experts").
 //
-// Router, per row, in float: z = W_r h, s = softmax(z) over all E experts (or, `logistic`, every
+// Router, per row, in float: z = W_r h (+ bias), s = softmax(z) over all E experts (or, `logistic`, every
 // expert's own 1 / (1 + exp(-z))).  The choice goes by c = s, or c = s + correction[e] (which may be
 // negative).  The experts form `groups` equal groups of neighbours; a group's score is its largest
 // c, or the sum of its two largest (`two_largest`), and only experts of the `keep` best groups can be
@@ -28,6 +28,7 @@ struct RouteTerms {
   int normalise;
   float normalise_eps;
   float* shared_weight;      // [n] or null; with it the router's matrix has a row E
+  const float* bias;         // [E] on the products, or null
 };
 
 template <typename T, int NT>
@@ -68,7 +69,7 @@ route_kernel(const T* __restrict__ h, int W, const float* __restrict__ wr, int E
       for (c = lane; c < W; c += WAVE) d0 = fmaf(w[c], to_f32(row[c]), d0);
     }
     float dot = wave_sum((d0 + d1) + (d2 + d3));
-    if (lane == 0) s_s[e] = dot;
+    if (lane == 0) s_s[e] = dot + (k.bias && e < E ? k.bias[e] : 0.f);
   }
   __syncthreads();
   if (k.shared_weight && t == 0) k.shared_weight[n] = 1.0f / (1.0f + expf(-s_s[E]));
@@ -372,8 +373,8 @@ using namespace tl;
 extern "C" {
 
 int tl_route(const void* h, int dt, int n, int W, const float* wr, int E, int groups, int keep, int top, int logistic,
-             const float* correction, int two_largest, int normalise, float normalise_eps, float* shared_weight, float* weights,
-             int* chosen, hipStream_t st) {
+             const float* correction, int two_largest, int normalise, float normalise_eps, float* shared_weight,
+             const float* bias, float* weights, int* chosen, hipStream_t st) {
   TL_REQUIRE(n >= 0 && W > 0 && E > 0 && E <= RT_MAX_E && top > 0 && top <= E, "route: bad sizes n=%d W=%d E=%d top=%d (experts up to %d)",
              n, W, E, top, RT_MAX_E);
   TL_REQUIRE(groups >= 0 && (groups == 0 || (E % groups == 0 && keep > 0 && keep <= groups && keep * (E / groups) >= top)),
@@ -382,7 +383,7 @@ int tl_route(const void* h, int dt, int n, int W, const float* wr, int E, int gr
   if (n == 0) return 0;
   const bool vec = W % 4 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)wr % 16 == 0;
   TL_REQUIRE(dt == DT_F32 || dt == DT_BF16, "route: unknown dtype code %d", dt);
-  const RouteTerms k{correction, two_largest, normalise, normalise_eps, shared_weight};
+  const RouteTerms k{correction, two_largest, normalise, normalise_eps, shared_weight, bias};
   const bool few = n <= 64 && E > 4;             // fewer rows than compute units: more waves a row
   if (dt == DT_F32 && few)
     route_kernel<float, 1024><<<n, 1024, 0, st>>>((const float*)h, W, wr, E, groups, keep, top, logistic, k, weights, chosen, vec);

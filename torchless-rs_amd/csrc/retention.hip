@@ -139,11 +139,12 @@ retention_scan_kernel(const float* __restrict__ proj, int width, int H, int dk, 
   }
 }
 
-// out[n, h, :] = o / sqrt(mean(o^2) + eps) * silu(g), one wave a head of a row
+// out[n, h, :] = factor * o / sqrt(mean(o^2) + eps) * w * (silu or logistic of g), one wave a head of a row; w (shared by
+// the heads) may be null
 template <typename T>
 __global__ void __launch_bounds__(256)
-retention_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ gate, int gate_stride, int H, int dv,
-                           float eps, int units, T* __restrict__ out) {
+heads_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w, const float* __restrict__ gate, int gate_stride, int silu,
+                       int H, int dv, float eps, float factor, int units, T* __restrict__ out, int out_stride) {
   const int unit = blockIdx.x * 4 + threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   if (unit >= units) return;
   const int n = unit / H, h = unit % H;
@@ -151,10 +152,11 @@ retention_norm_gate_kernel(const float* __restrict__ o, const float* __restrict_
   const float* gr = gate + (size_t)n * gate_stride + (size_t)h * dv;
   float ss = 0.f;
   for (int c = lane; c < dv; c += WAVE) ss += row[c] * row[c];
-  const float f = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
+  const float f = factor / sqrtf(wave_sum(ss) / (float)dv + eps);
   for (int c = lane; c < dv; c += WAVE) {
     const float a = gr[c];
-    out[((size_t)n * H + h) * dv + c] = from_f32<T>(row[c] * f * (a / (1.0f + expf(-a))));
+    out[(size_t)n * out_stride + (size_t)h * dv + c] =
+        from_f32<T>(row[c] * f * (w ? w[c] : 1.f) * ((silu ? a : 1.0f) / (1.0f + expf(-a))));
   }
 }
 
@@ -223,20 +225,22 @@ int tl_retention_scan(const float* proj, int width, int H, int dk, int dv, const
   return 0;
 }
 
-// o float [n, H*dv]; gate: the column of the first gate channel in a row of `gate_stride` floats
-int tl_retention_norm_gate(const float* o, const float* gate, int gate_stride, int n, int H, int dv, float eps, void* out,
-                           int dt, hipStream_t st) {
-  TL_REQUIRE(n >= 0 && H > 0 && dv > 0 && gate_stride >= H * dv, "retention_norm_gate: bad sizes n=%d H=%d dv=%d", n, H, dv);
-  TL_REQUIRE(o && gate && out, "retention_norm_gate: a buffer is missing");
-  TL_REQUIRE((long long)n * H < 2147483647LL, "retention_norm_gate: too many heads");
-  TL_REQUIRE(dt == DT_F32 || dt == DT_BF16, "retention_norm_gate: unknown dtype code %d", dt);
+// o float [n, H*dv]; gate: the column of the first gate channel in a row of `gate_stride` floats; w [dv] or null
+int tl_heads_norm_gate(const float* o, const float* w, const float* gate, int gate_stride, int silu, int n, int H, int dv, float eps,
+                       float factor, void* out, int out_stride, int dt, hipStream_t st) {
+  TL_REQUIRE(n >= 0 && H > 0 && dv > 0 && gate_stride >= H * dv && out_stride >= H * dv, "heads_norm_gate: bad sizes n=%d H=%d dv=%d", n, H, dv);
+  TL_REQUIRE(o && gate && out, "heads_norm_gate: a buffer is missing");
+  TL_REQUIRE((long long)n * H < 2147483647LL, "heads_norm_gate: too many heads");
+  TL_REQUIRE(dt == DT_F32 || dt == DT_BF16, "heads_norm_gate: unknown dtype code %d", dt);
   if (n == 0) return 0;
   const int units = n * H;
   if (dt == DT_F32)
-    retention_norm_gate_kernel<float><<<(units + 3) / 4, 256, 0, st>>>(o, gate, gate_stride, H, dv, eps, units, (float*)out);
+    heads_norm_gate_kernel<float><<<(units + 3) / 4, 256, 0, st>>>(o, w, gate, gate_stride, silu, H, dv, eps, factor, units, (float*)out,
+                                                                  out_stride);
   else
-    retention_norm_gate_kernel<bf16><<<(units + 3) / 4, 256, 0, st>>>(o, gate, gate_stride, H, dv, eps, units, (bf16*)out);
-  TL_LAUNCH_CHECK("retention_norm_gate");
+    heads_norm_gate_kernel<bf16><<<(units + 3) / 4, 256, 0, st>>>(o, w, gate, gate_stride, silu, H, dv, eps, factor, units, (bf16*)out,
+                                                                 out_stride);
+  TL_LAUNCH_CHECK("heads_norm_gate");
   return 0;
 }
 

@@ -369,6 +369,20 @@ int tl_ssm_conv(const float* proj, int width, int off, int C, const float* w, co
   return 0;
 }
 
+// The last taps - 1 rows of the columns off .. off + C - 1 of every sequence's rows, kept for its next step: for a mixer whose
+// own kernel does the convolution of several rows.
+int tl_conv_carry(const float* proj, int width, int off, int C, int taps, float* conv_state, long long stride, const int* cu_seqlens,
+                  const int* slots, int B, hipStream_t st) {
+  TL_REQUIRE(B >= 0 && C > 0 && off >= 0 && off + C <= width && taps >= 1 && taps <= SSM_MAX_TAPS, "conv_carry: bad sizes C=%d off=%d width=%d taps=%d",
+             C, off, width, taps);
+  TL_REQUIRE(proj && conv_state && cu_seqlens && slots, "conv_carry: a buffer is missing");
+  TL_REQUIRE(stride >= (long long)(taps - 1) * C, "conv_carry: a sequence's block is too small for %d rows of %d", taps - 1, C);
+  if (B == 0 || taps == 1) return 0;
+  ssm_conv_carry_kernel<<<dim3(B, (C + 255) / 256), 256, 0, st>>>(proj, width, off, C, taps, conv_state, stride, cu_seqlens, slots);
+  TL_LAUNCH_CHECK("conv_carry");
+  return 0;
+}
+
 // u [n, C] = [x | B | C] after the convolution; proj [n, width] holds dt at column dt_off + h.
 int tl_ssm_scan(const void* u, int dt, int C, int G, int N, int heads, int dv, const float* proj, int width, int dt_off,
                 const float* dt_bias, const float* A_log, const float* D, float* state, long long stride,

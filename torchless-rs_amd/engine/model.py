@@ -18,6 +18,9 @@ from ..parts.base import ModelSpec, PartSpec, RunBinding, StepContext, flush_pen
 from ..weights.binding import bind_weights
 
 
+EMBEDDING_RUN = -1            # the number under which the cache keeps the embedding's state, beside those of the runs
+
+
 class Model:
     def __init__(self, spec: ModelSpec, config: Optional[ModelConfig], dtype: torch.dtype, device):
         if dtype not in (torch.float32, torch.bfloat16):
@@ -90,6 +93,9 @@ class Model:
     def cache_requests(self):
         kv: Dict[int, KVRequest] = {}
         st: Dict[int, StateRequest] = {}
+        keeps = getattr(self.embedding, "state_request", None)
+        if keeps is not None and keeps() is not None:
+            st[EMBEDDING_RUN] = keeps()
         for i, run in enumerate(self.spec.schedule):
             mixer = self.blocks[run.layer].mixer
             if run.kv_from is None:
@@ -137,11 +143,15 @@ class Model:
         H, V = self.spec.hidden_size, self.spec.vocab_size
         ws = ctx.workspace
         x = ws.get("residual", (ctx.n_rows, H), torch.float32)
-        self.embedding.forward(ctx, ctx.tokens, x)
+        state = ctx.cache.state.get(EMBEDDING_RUN) if ctx.cache is not None else None
+        if state is None:
+            self.embedding.forward(ctx, ctx.tokens, x)
+        else:
+            self.embedding.forward(ctx, ctx.tokens, x, state)
         embedded = None
         if any(p.needs_embedding for p in self.stream_parts):      # someone adds the embedding's output again later
             embedded = ws.get("embedded", (ctx.n_rows, H), torch.float32)
-            self.embedding.forward(ctx, ctx.tokens, embedded)
+            embedded.copy_(x)
         schedule = self.spec.schedule
         order = [self.blocks[run.layer] for run in schedule]
         handed = False                       # the block before saw to this run's stream part

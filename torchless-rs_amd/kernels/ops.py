@@ -87,6 +87,44 @@ def embed(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scale: floa
     _check(lib().tl_embed(_p(table), _code(table.dtype), _p(ids), n, H, ctypes.c_float(scale), _p(out), _stream()))
 
 
+class PairTable:
+    """A second embedding table read by pairs of tokens: row (previous * mul_prev + current * mul_cur) mod `buckets` of `table`
+    [buckets + 1, H]; a sequence's first token reads the last row.  The previous token of a sequence's first row of
+    a step is what the step before left in the sequence's block."""
+
+    def __init__(self, table: torch.Tensor, buckets: int, mul_prev: int, mul_cur: int):
+        self.table, self.buckets = table, int(buckets)
+        self.mul_prev, self.mul_cur = int(mul_prev) % self.buckets, int(mul_cur) % self.buckets     # (the same rows, smaller products)
+
+
+def embed_pairs(table: torch.Tensor, ids: torch.Tensor, scale: float, pairs: Optional[PairTable], row_pos, row_seq, cu_seqlens,
+                slots, last: Optional[torch.Tensor], norm_weight: Optional[torch.Tensor], eps: float, out: torch.Tensor) -> None:
+    """out[n, :] = table[ids[n], :] * scale, plus the pair's row (`pairs`), then divided by the row's root mean square and times
+    `norm_weight` (float32 [H]; None: no norm), all in float32.  `last` (int32 [slots, 1]): every sequence's last token, read for
+    its first row (unless that is position 0) and left behind by this step."""
+    n, H = ids.shape[0], table.shape[1]
+    B = slots.shape[0]
+    _req(table, "embed_pairs.table")
+    _req(ids, "embed_pairs.ids", torch.int32, (n,))
+    if pairs is not None:
+        _req(pairs.table, "embed_pairs.pairs", table.dtype, (pairs.buckets + 1, H))
+        _req(row_pos, "embed_pairs.row_pos", torch.int32, (n,))
+        _req(row_seq, "embed_pairs.row_seq", torch.int32, (n,))
+        _req(cu_seqlens, "embed_pairs.cu_seqlens", torch.int32, (B + 1,))
+        _req(slots, "embed_pairs.slots", torch.int32)
+        if last is None:
+            raise KernelError("embed_pairs: pairs need the sequences' last tokens")
+        _req(last, "embed_pairs.last", torch.int32, (last.shape[0], 1))
+    if norm_weight is not None:
+        _req(norm_weight, "embed_pairs.norm_weight", torch.float32, (H,))
+    _req(out, "embed_pairs.out", torch.float32, (n, H))
+    p = pairs
+    _check(lib().tl_embed_pairs(_p(table), _code(table.dtype), _p(ids), n, H, ctypes.c_float(scale), _p(p.table) if p else None,
+                                ctypes.c_longlong(p.buckets if p else 1), ctypes.c_longlong(p.mul_prev if p else 0),
+                                ctypes.c_longlong(p.mul_cur if p else 0), _p(row_pos), _p(row_seq), _p(cu_seqlens), _p(slots),
+                                _p(last), _p(norm_weight), ctypes.c_float(eps), _p(out), _stream()))
+
+
 def rmsnorm_add(z: torch.Tensor, w: torch.Tensor, eps: float, x: torch.Tensor, w_next: Optional[torch.Tensor] = None,
                 eps_next: float = 0.0, out: Optional[torch.Tensor] = None) -> None:
     """The RMS norm of a sublayer's output added to the stream: x += z / sqrt(mean(z^2) + eps) * w
@@ -642,7 +680,7 @@ class ProjectionTerms:
 
 def split_projection(proj: torch.Tensor, row_pos, terms: ProjectionTerms, nq: int, nkv: int, dk: int, dv: int,
                      ng: int, q: torch.Tensor, k, v, gate, table=None, ring_pages: int = 0, pages=None) -> None:
-    """proj float32 [n, nq*dk + nkv*(dk+dv) + ng] -> q [n, nq, dk], gate float32 [n, ng] (after the
+    """proj float32 [n, nq*dk + nkv*(dk+dv) + ng] (rows may be strided: columns of a wider product) -> q [n, nq, dk], gate float32 [n, ng] (after the
     logistic function) and, with nkv > 0, k [n, nkv, dk] and v [n, nkv, dv], or, with `pages`
     (one token a sequence, row n belongs to sequence n), k and v straight into the page of the
     row's position."""
@@ -798,18 +836,19 @@ class HeadTerms:
     square (eps inside the root) times a weight that all heads share; `mix`: 0, or 1 (the values
     are left, unrounded, for later layers) or 2 (v <- (1 - lam) v + lam * the values that were left);
     `unit_norm`: instead of the weighted norm, every head of q and of k is divided by its root mean
-    square (the same eps) AFTER the rotation, with no weight."""
+    square (the same eps) AFTER the rotation, with no weight; `v_factor` multiplies the (biased) values."""
 
     def __init__(self, bias=None, q_norm=None, k_norm=None, eps: float = 0.0, mix: int = 0, lam: float = 0.0,
-                 unit_norm: bool = False):
+                 unit_norm: bool = False, v_factor: float = 1.0):
         self.bias, self.q_norm, self.k_norm, self.eps = bias, q_norm, k_norm, float(eps)
         self.mix, self.lam = int(mix), float(lam)
         self.unit_norm = bool(unit_norm)
+        self.v_factor = float(v_factor)
 
 
 def head_prepare(proj: torch.Tensor, row_pos, rotation, terms: HeadTerms, nq: int, nkv: int, dk: int, dv: int, ng: int,
                  q: torch.Tensor, k, v, gate, v_first=None, table=None, ring_pages: int = 0, pages=None) -> None:
-    """proj float32 [n, nq*dk + nkv*(dk+dv) + ng] -> q [n, nq, dk] (biased, normed per head, rotated),
+    """proj float32 [n, nq*dk + nkv*(dk+dv) + ng] (rows may be strided: columns of a wider product) -> q [n, nq, dk] (biased, normed per head, rotated),
     `gate` float32 [n, ng] (after the logistic function) and k [n, nkv, dk] and v [n, nkv, dv], or,
     with `pages` (one token a sequence, row n belongs to sequence n), k and v straight into the
     page of the row's position.  `v_first` (float32 [n, nkv*dv]): where a layer that mixes values
@@ -820,7 +859,7 @@ def head_prepare(proj: torch.Tensor, row_pos, rotation, terms: HeadTerms, nq: in
     rot = _rotation(rotation, dk, "head_prepare")
     if rot.interleaved:
         raise KernelError("head_prepare: pairs (2i, 2i + 1) are not served, only (i, i + rotary_dim / 2)")
-    _req(proj, "head_prepare.proj", torch.float32, (n, width))
+    _req_columns(proj, (n, width), "head_prepare.proj")
     _req(row_pos, "head_prepare.row_pos", torch.int32, (n,))
     _req(q, "head_prepare.q", None, (n, nq, dk))
     for t, name, size in ((terms.bias, "bias", width), (terms.q_norm, "q_norm", dk), (terms.k_norm, "k_norm", dk)):
@@ -844,9 +883,10 @@ def head_prepare(proj: torch.Tensor, row_pos, rotation, terms: HeadTerms, nq: in
         if pages.dtype != q.dtype or table.dim() != 2 or table.shape[0] != n:
             raise KernelError("head_prepare: pages of q's dtype and a page table with one row per row")
         stride = table.shape[1]
-    _check(lib().tl_head_prepare(_p(proj), _p(row_pos), _p(rot.inv_freq), rot.rotary_dim, _p(terms.bias), _p(terms.q_norm),
+    _check(lib().tl_head_prepare(_p(proj), proj.stride(0), _p(row_pos), _p(rot.inv_freq), rot.rotary_dim, _p(terms.bias), _p(terms.q_norm),
                                  _p(terms.k_norm), ctypes.c_float(terms.eps), int(terms.unit_norm), terms.mix,
-                                 ctypes.c_float(terms.lam), _p(v_first) if terms.mix else None, n, nq, nkv, dk, dv, ng, _p(q),
+                                 ctypes.c_float(terms.lam), ctypes.c_float(terms.v_factor),
+                                 _p(v_first) if terms.mix else None, n, nq, nkv, dk, dv, ng, _p(q),
                                  _p(k) if pages is None else None, _p(v) if pages is None else None, _p(gate),
                                  _code(q.dtype), _p(table), stride, int(ring_pages), _p(pages), _stream()))
 
@@ -942,8 +982,8 @@ def _shared_weight(w: Optional[torch.Tensor], n: int, what: str):
 def route(h: torch.Tensor, router: torch.Tensor, groups: int, keep: int, top: int, weights: torch.Tensor,
           chosen: Optional[torch.Tensor] = None, logistic: bool = False, correction: Optional[torch.Tensor] = None,
           two_largest: bool = False, normalise_eps: Optional[float] = None,
-          shared_weight: Optional[torch.Tensor] = None) -> None:
-    """The router of a mixture of experts, in float32: s = softmax(router h) over the E experts (`logistic`:
+          shared_weight: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> None:
+    """The router of a mixture of experts, in float32: s = softmax(router h (+ `bias`, float32 [E])) over the E experts (`logistic`:
     every expert's own 1 / (1 + exp(-router h)) instead).  The choice goes by c = s (+ `correction`, float32 [E]):
     of the `keep` groups (of `groups` equal groups of neighbours; 0: no groups) whose best c is largest
     (`two_largest`: the sum of whose two best is), the `top` experts with the largest c; `weights` float32
@@ -959,10 +999,12 @@ def route(h: torch.Tensor, router: torch.Tensor, groups: int, keep: int, top: in
         _req(chosen, "route.chosen", torch.int32, (n, top))
     if correction is not None:
         _req(correction, "route.correction", torch.float32, (E,))
+    if bias is not None:
+        _req(bias, "route.bias", torch.float32, (E,))
     _check(lib().tl_route(_p(h), _code(h.dtype), n, W, _p(router), E, int(groups), int(keep), int(top), int(bool(logistic)),
                           _p(correction), int(bool(two_largest)), int(normalise_eps is not None),
-                          ctypes.c_float(normalise_eps or 0.0), _shared_weight(shared_weight, n, "route"), _p(weights),
-                          _p(chosen), _stream()))
+                          ctypes.c_float(normalise_eps or 0.0), _shared_weight(shared_weight, n, "route"), _p(bias),
+                          _p(weights), _p(chosen), _stream()))
 
 
 class GateTerms:
@@ -1311,16 +1353,30 @@ def retention_scan(proj: torch.Tensor, row_pos, rotation, H: int, dk: int, dv: i
                                    _stream()))
 
 
-def retention_norm_gate(o: torch.Tensor, gate: torch.Tensor, H: int, eps: float, out: torch.Tensor) -> None:
-    """out[n, h] = o / sqrt(mean(o^2) + eps) * silu(gate) per head: o float32 [n, H*dv], gate float32 [n, H*dv] (rows may
-    be strided: columns of the projection), out in the compute dtype."""
+def _req_columns(t: torch.Tensor, shape, what: str, dtype=torch.float32) -> None:
+    """Columns of a wider matrix: rows may be strided."""
+    if not t.is_cuda or t.dtype != dtype or tuple(t.shape) != tuple(shape) or t.stride(1) != 1:
+        raise KernelError(f"{what}: {dtype} {list(shape)} on the GPU, rows may be strided")
+
+
+def heads_norm_gate(o: torch.Tensor, gate: torch.Tensor, H: int, eps: float, out: torch.Tensor, weight: Optional[torch.Tensor] = None,
+                    silu: bool = True, factor: float = 1.0) -> None:
+    """out[n, h] = factor * o / sqrt(mean(o^2) + eps) * weight * silu(gate) (`silu` False: its logistic function) per head: o
+    float32 [n, H*dv], gate float32 [n, H*dv] (rows may be strided: columns of the projection), weight float32 [dv] that all
+    heads share (None: none), out [n, H*dv] in the compute dtype (rows may be strided)."""
     n, inner = o.shape
-    _req(o, "retention_norm_gate.o", torch.float32)
-    if gate.dtype != torch.float32 or tuple(gate.shape) != (n, inner) or gate.stride(1) != 1 or not gate.is_cuda:
-        raise KernelError(f"retention_norm_gate.gate: float32 [{n}, {inner}] on the GPU, rows may be strided")
-    _req(out, "retention_norm_gate.out", None, (n, inner))
-    _check(lib().tl_retention_norm_gate(_p(o), _p(gate), gate.stride(0), n, H, inner // H, ctypes.c_float(eps), _p(out),
-                                        _code(out.dtype), _stream()))
+    _req(o, "heads_norm_gate.o", torch.float32)
+    _req_columns(gate, (n, inner), "heads_norm_gate.gate")
+    if weight is not None:
+        _req(weight, "heads_norm_gate.weight", torch.float32, (inner // H,))
+    _req_columns(out, (n, inner), "heads_norm_gate.out", out.dtype)
+    _check(lib().tl_heads_norm_gate(_p(o), _p(weight), _p(gate), gate.stride(0), int(bool(silu)), n, H, inner // H, ctypes.c_float(eps),
+                                    ctypes.c_float(factor), _p(out), out.stride(0), _code(out.dtype), _stream()))
+
+
+def retention_norm_gate(o: torch.Tensor, gate: torch.Tensor, H: int, eps: float, out: torch.Tensor) -> None:
+    """`heads_norm_gate` as retention has it: no weight, silu."""
+    heads_norm_gate(o, gate, H, eps, out)
 
 
 def retention_chunk() -> int:
@@ -1360,6 +1416,118 @@ def retention_chunks(proj: torch.Tensor, row_pos, rotation, H: int, dk: int, dv:
                                      int(rot.interleaved), ctypes.c_float(rot.magnitude), ctypes.c_float(kscale), _p(log2_decay),
                                      ctypes.c_float(eps), _p(state), ctypes.c_longlong(state.stride(0)), _p(cu_seqlens), _p(slots), n,
                                      B, int(chunks), *[_p(t) for t in scratch], _p(out), _stream()))
+
+
+# ---- linear attention with a decay per key channel -----------------------------------------------------
+class ChannelTerms:
+    """How a row of a product becomes the rows of a linear attention with a decay per head and key channel: `G` heads of q and
+    k, `H` of v and of the decays, sizes dk and dv; columns of beta (`b_off`, None: the plain recurrence, no delta rule), of the
+    decays' inner row (`a_off`, `a_rank` channels; second matrix `a2` [H*dk, a_rank], `bias` float32 [H*dk] or None) and of the
+    gate's (`g_off`, `g_rank`, `g2` [H*dv, g_rank]; None: the gate is none of this); `conv` (float32 [2*G*dk + H*dv, taps], None:
+    no convolution); `rate` (float32 [H]: decays exp(-exp(rate) softplus(z)); None: logistic(z)^(1 / tau)); `qscale`; `unit_eps`
+    (None: q and k are not made unit vectors)."""
+
+    def __init__(self, G: int, H: int, dk: int, dv: int, a_off: int, a2: torch.Tensor, bias=None, b_off: Optional[int] = None,
+                 g_off: Optional[int] = None, g2: Optional[torch.Tensor] = None, conv: Optional[torch.Tensor] = None,
+                 rate: Optional[torch.Tensor] = None, tau: float = 1.0, qscale: float = 1.0, unit_eps: Optional[float] = None):
+        self.G, self.H, self.dk, self.dv = int(G), int(H), int(dk), int(dv)
+        self.a_off, self.a2, self.bias, self.b_off, self.g_off, self.g2 = int(a_off), a2, bias, b_off, g_off, g2
+        self.conv, self.rate, self.inv_tau, self.qscale, self.unit_eps = conv, rate, 1.0 / float(tau), float(qscale), unit_eps
+
+    @property
+    def channels(self) -> int:
+        """The columns [q | k | v] that a convolution covers."""
+        return 2 * self.G * self.dk + self.H * self.dv
+
+    @property
+    def taps(self) -> int:
+        return 0 if self.conv is None else int(self.conv.shape[1])
+
+    def check(self, what: str) -> None:
+        _req(self.a2, what + ".a2", None, (self.H * self.dk, self.a2.shape[1]))
+        if self.g2 is not None:
+            _req(self.g2, what + ".g2", self.a2.dtype, (self.H * self.dv, self.g2.shape[1]))
+        if self.bias is not None:
+            _req(self.bias, what + ".bias", torch.float32, (self.H * self.dk,))
+        if self.rate is not None:
+            _req(self.rate, what + ".rate", torch.float32, (self.H,))
+        if self.conv is not None:
+            _req(self.conv, what + ".conv", torch.float32, (self.channels, self.taps))
+
+
+def channel_rows(proj: torch.Tensor, t: ChannelTerms, conv_state, row_seq, cu_seqlens, slots, single: bool, q, k, v, decay, beta,
+                 gate) -> None:
+    """proj float32 [n, width] (rows may be strided) = [q | k | v | ...] -> q, k float32 [n, G*dk], v [n, H*dv], decay [n, H*dk]
+    (factors between 0 and 1), beta [n, H] (with the delta rule) and gate [n, H*dv] (second step of its projection, where the
+    terms have one): see `ChannelTerms`.  `conv_state` (float32 [slots, >= (taps - 1) * channels]): the convolution's last
+    inputs, read and left updated."""
+    n, width = proj.shape
+    B = slots.shape[0]
+    _req_columns(proj, (n, width), "channel_rows.proj")
+    t.check("channel_rows")
+    for x, name, size in ((q, "q", t.G * t.dk), (k, "k", t.G * t.dk), (v, "v", t.H * t.dv), (decay, "decay", t.H * t.dk),
+                          (beta, "beta", t.H), (gate, "gate", t.H * t.dv)):
+        if (name == "beta" and t.b_off is None) or (name == "gate" and t.g2 is None):
+            continue
+        _req(x, "channel_rows." + name, torch.float32, (n, size))
+    if t.taps:
+        _req_state(conv_state, (t.taps - 1) * t.channels, "channel_rows")
+        _req(row_seq, "channel_rows.row_seq", torch.int32, (n,))
+    _req(cu_seqlens, "channel_rows.cu_seqlens", torch.int32, (B + 1,))
+    _req(slots, "channel_rows.slots", torch.int32)
+    if proj.shape[1] < t.channels:
+        raise KernelError(f"channel_rows: rows of {width} for {t.channels} channels")
+    _check(lib().tl_channel_rows(_p(proj), proj.stride(0), t.G, t.H, t.dk, t.dv, -1 if t.b_off is None else int(t.b_off), t.a_off,
+                                 t.a2.shape[1], 0 if t.g2 is None else int(t.g_off), 0 if t.g2 is None else t.g2.shape[1], t.taps,
+                                 _p(t.conv), _p(t.bias), _p(t.rate), ctypes.c_float(t.inv_tau), ctypes.c_float(t.qscale),
+                                 ctypes.c_float(-1.0 if t.unit_eps is None else t.unit_eps), _p(t.a2), _p(t.g2), _code(t.a2.dtype),
+                                 _p(conv_state), ctypes.c_longlong(conv_state.stride(0) if t.taps else 0), _p(row_seq),
+                                 _p(cu_seqlens), _p(slots), n, B, int(bool(single)), _p(q), _p(k), _p(v), _p(decay), _p(beta),
+                                 _p(gate), _stream()))
+    if t.taps and not single:
+        conv_carry(proj, 0, t.channels, t.taps, conv_state, cu_seqlens, slots)
+
+
+def conv_carry(proj: torch.Tensor, off: int, C: int, taps: int, conv_state: torch.Tensor, cu_seqlens, slots) -> None:
+    """Keep the last taps - 1 rows of the columns off .. off + C - 1 of every sequence's rows in its block (older ones shifted
+    down where a step brings fewer)."""
+    _check(lib().tl_conv_carry(_p(proj), proj.stride(0), int(off), int(C), int(taps), _p(conv_state),
+                               ctypes.c_longlong(conv_state.stride(0)), _p(cu_seqlens), _p(slots), slots.shape[0], _stream()))
+
+
+def _channel_scan(q, k, v, decay, beta, t: ChannelTerms, state, cu_seqlens, slots, o, weight, gate, silu, eps, factor, out) -> None:
+    n, B = q.shape[0], slots.shape[0]
+    for x, name, size in ((q, "q", t.G * t.dk), (k, "k", t.G * t.dk), (v, "v", t.H * t.dv), (decay, "decay", t.H * t.dk)):
+        _req(x, "channel_scan." + name, torch.float32, (n, size))
+    if t.b_off is not None:
+        _req(beta, "channel_scan.beta", torch.float32, (n, t.H))
+    _req_state(state, t.H * t.dk * t.dv, "channel_scan")
+    _req(cu_seqlens, "channel_scan.cu_seqlens", torch.int32, (B + 1,))
+    _req(slots, "channel_scan.slots", torch.int32)
+    _check(lib().tl_channel_scan(_p(q), _p(k), _p(v), _p(decay), _p(beta) if t.b_off is not None else None, t.G, t.H, t.dk, t.dv,
+                                 _p(state), ctypes.c_longlong(state.stride(0)), _p(cu_seqlens), _p(slots), n, B, _p(o), _p(weight),
+                                 _p(gate), gate.stride(0) if gate is not None else 0, int(bool(silu)), ctypes.c_float(eps),
+                                 ctypes.c_float(factor), _p(out), out.stride(0) if out is not None else 0,
+                                 _code(out.dtype) if out is not None else DT_F32, _stream()))
+
+
+def channel_scan(q, k, v, decay, beta, t: ChannelTerms, state: torch.Tensor, cu_seqlens, slots, o: torch.Tensor) -> None:
+    """The recurrence row after row, sequence by sequence, all in float32, over what `channel_rows` made: `state` float32
+    [slots, >= H*dv*dk] (a head's state column by column) is read and left updated; o float32 [n, H*dv]."""
+    _req(o, "channel_scan.o", torch.float32, (q.shape[0], t.H * t.dv))
+    _channel_scan(q, k, v, decay, beta, t, state, cu_seqlens, slots, o, None, None, True, 0.0, 1.0, None)
+
+
+def channel_scan_gated(q, k, v, decay, beta, t: ChannelTerms, state: torch.Tensor, cu_seqlens, slots, gate: torch.Tensor, eps: float,
+                       out: torch.Tensor, weight=None, silu: bool = True, factor: float = 1.0) -> None:
+    """`channel_scan` and `heads_norm_gate` of a step in which every sequence brings one row (row b is sequence b's), in one
+    kernel."""
+    n, inner = q.shape[0], t.H * t.dv
+    _req_columns(gate, (n, inner), "channel_scan.gate")
+    _req_columns(out, (n, inner), "channel_scan.out", out.dtype)
+    if weight is not None:
+        _req(weight, "channel_scan.weight", torch.float32, (t.dv,))
+    _channel_scan(q, k, v, decay, beta, t, state, cu_seqlens, slots, None, weight, gate, silu, eps, factor, out)
 
 
 def take_tokens(src: torch.Tensor, idx: torch.Tensor, vocab: int, tokens: torch.Tensor) -> None:

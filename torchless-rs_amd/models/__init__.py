@@ -9,6 +9,7 @@ from . import fanitar as _fanitar         # registers Fanitar
 from . import nepisun as _nepisun         # registers Nepisun
 from . import giforax as _giforax         # registers Giforax
 from . import zudalorn as _zudalorn       # registers Zudalorn
+from . import zifetar as _zifetar         # registers Zifetar
 
 
 def model_spec_for(cfg: ModelConfig):

@@ -2,7 +2,7 @@
 
 Every mechanism is a constructor parameter and can be left out:
 
-* biases on the q, k, v and o projections (`bias`);
+* biases on the q, k, v and o projections (`bias`; `o_bias` False: on q, k and v alone);
 * a norm of q and of k PER HEAD: every head divided by its own root mean square over its
   channels (eps inside the root) times a weight of one head's size that all heads share
   (`head_norm_eps`; None: none), before the rotation;
@@ -47,13 +47,13 @@ from ..cache.cache import KVRequest
 from ..kernels import ops
 from ..weights.binding import WeightSpec
 from .attention_scored import attend_and_commit
-from .base import Mixer, PartSpec, flush_pending, make_part, register_part
-from .linear import Linear
+from .base import PartSpec, flush_pending, make_part, register_part
+from .projected import ProjectedMixer
 
 VALUE_MIX = (None, "first", "later")
 
 
-class HeadwiseAttentionMixer(Mixer):
+class HeadwiseAttentionMixer(ProjectedMixer):
     graph_safe = True
 
     NAMES = {"q": "q", "k": "k", "v": "v", "o": "o", "q_bias": "q.b", "k_bias": "k.b", "v_bias": "v.b",
@@ -65,7 +65,7 @@ class HeadwiseAttentionMixer(Mixer):
                  keep_first: int = 0, unit_sink: bool = False, channel_gate: bool = False,
                  value_mix: Optional[str] = None, prefix: str = "mix.", names: Optional[Dict[str, str]] = None,
                  unit_norm_eps: Optional[float] = None, chunk: Optional[int] = None, logistic: bool = False,
-                 head_gate: bool = False, own_kv: bool = True):
+                 head_gate: bool = False, own_kv: bool = True, o_bias: Optional[bool] = None):
         if n_heads % n_kv_heads:
             raise ValueError(f"attention: {n_heads} heads are not a multiple of {n_kv_heads} KV heads")
         if value_mix not in VALUE_MIX:
@@ -80,6 +80,7 @@ class HeadwiseAttentionMixer(Mixer):
         self.position = make_part("position", position if position is not None else PartSpec("none"))
         self.scale = 1.0 / math.sqrt(self.dk) if scale is None else float(scale)
         self.bias = bool(bias)
+        self.has_o_bias = self.bias if o_bias is None else bool(o_bias)
         self.head_norm_eps = None if head_norm_eps is None else float(head_norm_eps)
         self.window = int(window) if window else None
         self.keep_first = int(keep_first) if self.window else 0
@@ -99,9 +100,10 @@ class HeadwiseAttentionMixer(Mixer):
             raise ValueError("attention: logistic weights have no denominator for one more to count in")
         if not self.own_kv and self.value_mix is not None:
             raise ValueError("attention: a mixer that reads another's values has none to mix")
+        self.tag = "hattn"
         self.ng = self.nq * self.dv if self.channel_gate else (self.nq if self.head_gate else 0)
-        self.closes_stream = not self.bias        # without a bias its last write to the stream is `Linear.add_into`
-        self.proj = self.o = self.o_bias = None
+        self.closes_stream = not self.has_o_bias  # without that bias its last write to the stream is `Linear.add_into`
+        self.o_bias = None
         self.head_terms = self.terms = None
 
     # ---- what it keeps -------------------------------------------------------
@@ -118,9 +120,6 @@ class HeadwiseAttentionMixer(Mixer):
         if not self.own_kv:
             return None
         return KVRequest(self.nkv, self.dk, self.kv_reach(), None if self.dv == self.dk else self.dv)
-
-    def may_capture(self, n_rows: int) -> bool:
-        return self.proj is not None and self.proj.own_kernels(n_rows) and self.o.own_kernels(n_rows)
 
     # ---- weights -------------------------------------------------------------
     def weight_specs(self) -> Dict[str, WeightSpec]:
@@ -143,11 +142,11 @@ class HeadwiseAttentionMixer(Mixer):
         if self.ng:
             out[p + nm["gate"]] = WeightSpec((self.ng, self.H))
         out[p + nm["o"]] = WeightSpec((self.H, self.nq * self.dv))
-        if self.bias:
+        if self.has_o_bias:
             out[p + nm["o_bias"]] = WeightSpec((self.H,))
         return out
 
-    def load(self, tensors, compute_dtype) -> None:
+    def load_terms(self, tensors, compute_dtype):
         p, nm = self.prefix, self.names
 
         def t(key):
@@ -159,40 +158,41 @@ class HeadwiseAttentionMixer(Mixer):
         ws = [t("q")] + ([t("k"), t("v")] if self.own_kv else []) + ([t("gate")] if self.ng else [])
         if len({w.dtype for w in ws}) > 1:
             ws = [w.to(torch.float32) for w in ws]
-        self.proj = Linear(torch.cat(ws, dim=0), tiled=True)
-        self.o = Linear(t("o"), tiled=True)
         dev = ws[0].device
         bias = None
         if self.bias:
             bias = torch.cat([f32("q_bias")] + ([f32("k_bias"), f32("v_bias")] if self.own_kv else []) +
                              [torch.zeros(self.ng, dtype=torch.float32, device=dev)]).contiguous()
+        if self.has_o_bias:
             self.o_bias = f32("o_bias")
+        if self.factor != 1.0 and self.value_mix is not None:
+            raise ValueError("attention: a factor on the result goes into the values, which other layers read here")
         normed = self.head_norm_eps is not None
         lam = float(t("mix").to(torch.float32).item()) if self.value_mix == "later" else 0.0
         self.head_terms = ops.HeadTerms(bias=bias, q_norm=f32("q_norm") if normed else None,
                                         k_norm=f32("k_norm") if normed else None,
                                         eps=self.head_norm_eps or self.unit_norm_eps or 0.0,
                                         mix=VALUE_MIX.index(self.value_mix), lam=lam,
-                                        unit_norm=self.unit_norm_eps is not None)
+                                        unit_norm=self.unit_norm_eps is not None, v_factor=self.factor)
         sinks = torch.zeros(self.nq, dtype=torch.float32, device=dev) if self.unit_sink else None
         self.terms = ops.ScoreTerms(self.scale, self.window, None, sinks, keep_first=self.keep_first, chunk=self.chunk,
                                     logistic=self.logistic, score_bias=f32("score_bias") if self.logistic else None)
+        if not self.own_kv and self.factor != 1.0:
+            raise ValueError("attention: a factor on the result goes into the values, which are another layer's here")
+        self.in_width, self.heads_width = sum(w.shape[0] for w in ws), self.nq * self.dv
+        return torch.cat(ws, dim=0), t("o")
 
     # ---- one step --------------------------------------------------------------
-    def produce(self, ctx, run, y: torch.Tensor, out: Optional[torch.Tensor], x: Optional[torch.Tensor] = None):
-        """The mixer's result stored in `out` (float32 [n, H]), or with `out` None added to the
-        stream `x`; returns the bias of the output projection, which the caller adds (None
-        without biases)."""
-        n, nq, nkv, dk, dv, ng = y.shape[0], self.nq, self.nkv, self.dk, self.dv, self.ng
+    def heads(self, ctx, run, proj: torch.Tensor, out: torch.Tensor) -> None:
+        """The heads' weighted sums, gated, in `out` [n, nq * dv]."""
+        n, nq, nkv, dk, dv, ng = proj.shape[0], self.nq, self.nkv, self.dk, self.dv, self.ng
         ws = ctx.workspace
         group = run.kv_group
-        own = nkv if self.own_kv else 0
-        proj = ws.get("hattn_proj", (n, nq * dk + own * (dk + dv) + ng), torch.float32)
-        self.proj(y, proj)
-        rotation = self.position.rotation(y.device) or ops.NO_ROTATION
+        rotation = self.position.rotation(proj.device) or ops.NO_ROTATION
         q = ws.get("hattn_q", (n, nq, dk), ctx.dtype)
         gate = ws.get("hattn_gate", (n, ng), torch.float32) if ng else None
-        att = ws.get("hattn_out", (n, nq, dv), ctx.dtype)
+        whole = out.is_contiguous()
+        att = out.view(n, nq, dv) if whole else ws.get("hattn_out", (n, nq, dv), ctx.dtype)
         v_first = ws.get("hattn_v_first", (n, nkv * dv), torch.float32) if self.value_mix else None
         tag = f"_{run.index}" if run.kv_read_later else ""      # rows that a later run reads are nobody else's
         k = v = None
@@ -211,15 +211,18 @@ class HeadwiseAttentionMixer(Mixer):
                           own=self.own_kv)
         if self.channel_gate:
             ops.mul_gate(att, gate)
-        if out is None:
-            self.o.add_into(att.view(n, nq * dv), x, ctx, "hattn_o_parts")
-        else:
-            self.o(att.view(n, nq * dv), out)
+        if not whole:
+            out.copy_(att.view(n, nq * dv))
+
+    def produce(self, ctx, run, y: torch.Tensor, out: torch.Tensor):
+        """The mixer's result stored in `out` (float32 [n, H]); returns the bias of the output projection, which the
+        caller adds (None without one)."""
+        super().produce(ctx, run, y, out)
         return self.o_bias
 
     def forward(self, ctx, run, y: torch.Tensor, x: torch.Tensor) -> None:
-        if not self.bias:
-            self.produce(ctx, run, y, None, x)
+        if not self.has_o_bias:
+            super().forward(ctx, run, y, x)
             return
         flush_pending(ctx, x)
         z = ctx.workspace.get("hattn_z", tuple(x.shape), torch.float32)

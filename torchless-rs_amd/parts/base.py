@@ -204,6 +204,19 @@ class StreamPart(Part):
         raise NotImplementedError
 
 
+class Embedding(Part):
+    """The stream's first content.  `table` is the token table, for a head that is tied to it."""
+    table = None
+
+    def state_request(self):
+        """A `StateRequest` if the embedding keeps something per sequence (tokens before the present one)."""
+        return None
+
+    def forward(self, ctx: "StepContext", ids: torch.Tensor, x: torch.Tensor, state: Optional[torch.Tensor] = None) -> None:
+        """ids int32 [n] -> x float32 [n, H]; `state` [max_slots, *shape] if the embedding asked for one.  Called once a step."""
+        raise NotImplementedError
+
+
 class Position(Part):
     """A position encoding, as the attention mixer asks for it: how q and k are rotated."""
 

@@ -20,7 +20,8 @@ activation "silu" makes gated experts silu(gate t) * (up t), with no clamp and n
 the scores without it; choice scores may be negative); `group_score` "two_largest" scores a group by
 the sum of its two largest choice scores; `normalise_eps` divides the chosen experts' scores by (their
 sum + that number); `shared_gated` multiplies the shared expert's output by the logistic function of
-one more row of the router (tensor `shared.sg`).
+one more row of the router (tensor `shared.sg`).  `router_bias` adds a learned number per expert to the router's product; with
+`score` "softmax" and `normalise_eps` 0 the weights are the softmax over the chosen experts' logits alone.
 
 All experts run as ONE wide feed-forward: their up projections stacked by rows (the shared
 expert's behind them), the activation times the row's weight of the column's expert, which is
@@ -118,7 +119,7 @@ class RoutedExperts(FeedForward):
     # leaf names under `prefix`; "{e}" is the expert's number
     NAMES = {"router": "router", "up": "e{e}.up", "down": "e{e}.down", "shared_up": "shared.up",
              "shared_down": "shared.down", "gate": "e{e}.gate", "shared_gate": "shared.gate", "correction": "correction",
-             "shared_weight": "shared.sg"}
+             "shared_weight": "shared.sg", "router_bias": "router.b"}
     SCORES = ("softmax", "sigmoid")
     GROUP_SCORES = ("largest", "two_largest")
     GATED_ACTIVATION = "swish_clamped"
@@ -128,14 +129,16 @@ class RoutedExperts(FeedForward):
                  prefix: str = "mlp.", names: Optional[Dict[str, str]] = None, score: str = "softmax",
                  gated: bool = False, activation_constants: Optional[Dict[str, float]] = None,
                  shared_limit: Optional[float] = None, weight_on: str = "output", correction: bool = False,
-                 group_score: str = "largest", normalise_eps: Optional[float] = None, shared_gated: bool = False):
+                 group_score: str = "largest", normalise_eps: Optional[float] = None, shared_gated: bool = False,
+                 router_bias: bool = False):
         self.gated = bool(gated)
         if group_score not in self.GROUP_SCORES:
             raise ValueError(f"experts: a group's score is one of {self.GROUP_SCORES}, got {group_score!r}")
         self.has_correction, self.two_largest = bool(correction), group_score == "two_largest"
         self.normalise_eps = None if normalise_eps is None else float(normalise_eps)
         self.shared_gated = bool(shared_gated) and bool(shared_size)
-        self.correction = None
+        self.has_router_bias = bool(router_bias)
+        self.correction = self.router_bias = None
         if score not in self.SCORES:
             raise ValueError(f"experts: scores are one of {self.SCORES}, got {score!r}")
         if weight_on not in ("output", "input"):
@@ -183,6 +186,8 @@ class RoutedExperts(FeedForward):
             out[p + nm["up"].format(e=e)] = WeightSpec((self.ff, self.H))
             out[p + nm["down"].format(e=e)] = WeightSpec((self.H, self.ff))
         out[p + nm["router"]] = WeightSpec((self.E, self.H))
+        if self.has_router_bias:
+            out[p + nm["router_bias"]] = WeightSpec((self.E,))
         if self.has_correction:
             out[p + nm["correction"]] = WeightSpec((self.E,))
         if self.shared:
@@ -211,6 +216,8 @@ class RoutedExperts(FeedForward):
         if self.shared_gated:                                        # the shared expert's gate: one row more
             router.append(tensors[p + nm["shared_weight"]].to(torch.float32))
         self.router = torch.cat(router, dim=0).contiguous()
+        if self.has_router_bias:
+            self.router_bias = tensors[p + nm["router_bias"]].to(torch.float32).contiguous()
         if self.has_correction:
             self.correction = tensors[p + nm["correction"]].to(torch.float32).contiguous()
 
@@ -222,7 +229,7 @@ class RoutedExperts(FeedForward):
         shared_weight = ws.get("experts_sw", (n,), torch.float32) if self.shared_gated else None
         ops.route(y, self.router, self.groups, self.keep, self.top, weights, picked, logistic=self.logistic,
                   correction=self.correction, two_largest=self.two_largest, normalise_eps=self.normalise_eps,
-                  shared_weight=shared_weight)
+                  shared_weight=shared_weight, bias=self.router_bias)
         return weights, picked, shared_weight
 
     def few_rows(self, y: torch.Tensor) -> bool:

@@ -1,7 +1,7 @@
 """Norms over a row of the stream, in float32.
 
 RMSNorm: y = x / sqrt(mean(x^2) + eps) * w (src/kernels/mod.rs:558-568 of the
-reference; weight used as it is).  LayerNorm: y = (x - mean) / sqrt(var + eps) * w + b
+reference; weight used as it is, or stored as its difference from one).  LayerNorm: y = (x - mean) / sqrt(var + eps) * w + b
 with var the mean of the squared deviations, a weight and an optional bias."""
 from __future__ import annotations
 
@@ -18,20 +18,23 @@ class RMSNorm(Norm):
     graph_safe = True
     takes_pending = True        # adds partial products left in ctx.pending while it reads the stream
 
-    def __init__(self, size: int, eps: float, name: str = "weight", scalar: bool = False):
+    def __init__(self, size: int, eps: float, name: str = "weight", scalar: bool = False, around_zero: bool = False):
         """`name`: the weight's leaf name behind the norm's prefix ("" where the prefix is the tensor);
-        `scalar`: the weight is one number for all channels (a tensor without dimensions)."""
+        `scalar`: the weight is one number for all channels (a tensor without dimensions); `around_zero`: the
+        tensor holds the weight's difference from one."""
         self.size = int(size)
         self.eps = float(eps)
         self.name = name
         self.scalar = bool(scalar)
+        self.around_zero = bool(around_zero)
         self.weight = None
 
     def weight_specs(self) -> Dict[str, WeightSpec]:
-        return {self.name: WeightSpec(() if self.scalar else (self.size,), init="ones")}
+        return {self.name: WeightSpec(() if self.scalar else (self.size,), init="zeros" if self.around_zero else "ones")}
 
     def load(self, tensors, compute_dtype) -> None:
-        self.weight = tensors[self.name].to(torch.float32).expand(self.size).contiguous()
+        w = tensors[self.name].to(torch.float32)
+        self.weight = (1.0 + w if self.around_zero else w).expand(self.size).contiguous()
 
     def add_to(self, ctx, z: torch.Tensor, x: torch.Tensor, out=None, bias=None, then=None) -> None:
         """x += norm(z + bias) in one kernel.  `then` = (norm, buffer): the norm that reads the

@@ -23,10 +23,19 @@ import torch
 
 @dataclass(frozen=True)
 class WeightSpec:
-    """What a part expects under one name."""
+    """What a part expects under one name.  The sizes of the dimensions listed in `free` are the
+    checkpoint's own affair (an inner size that no configuration names); `shape` then holds what random
+    weights get there."""
     shape: Tuple[int, ...]
     integer: bool = False
-    init: str = "normal"      # how random weights fill it: "normal", "ones" (norm weights) or "mean" (weights of an average)
+    # how random weights fill it: "normal", "ones" (norm weights), "zeros" (norm weights kept as the difference from one) or
+    # "mean" (weights of an average)
+    init: str = "normal"
+    free: Tuple[int, ...] = ()
+
+    def fits(self, shape: Sequence[int]) -> bool:
+        return len(shape) == len(self.shape) and all(
+            (g >= 1 if i in self.free else g == w) for i, (g, w) in enumerate(zip(shape, self.shape)))
 
 
 class WeightBindingError(ValueError):
@@ -77,7 +86,7 @@ def bind_weights(expected: Dict[str, WeightSpec], source, compute_dtype: torch.d
         if n not in have:
             continue
         got = tuple(source.shape(n))
-        if got != tuple(spec.shape):
+        if not spec.fits(got):
             mismatched.append((n, got, tuple(spec.shape)))
         dt = source.dtype(n)
         if spec.integer and dt.is_floating_point:

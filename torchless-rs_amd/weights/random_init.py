@@ -28,8 +28,8 @@ def random_tensors(expected: Dict[str, WeightSpec], seed: int, std: float = 0.02
     for name, spec in expected.items():
         if spec.integer:
             out[name] = torch.zeros(spec.shape, dtype=torch.int32, device=device)
-        elif spec.init == "ones":
-            t = torch.ones(spec.shape, dtype=torch.float32, device=device)
+        elif spec.init in ("ones", "zeros"):
+            t = (torch.ones if spec.init == "ones" else torch.zeros)(spec.shape, dtype=torch.float32, device=device)
             if norm_std:
                 t += norm_std * torch.randn(spec.shape, generator=gen, dtype=torch.float32,
                                             device=device)
