@@ -300,6 +300,72 @@ def zudalorn_counts(z: dict, layers: int, B: int, C: int, T: int):
     return w, kv, att, w_read
 
 
+def zifetar_layers(layers: int):
+    """The mixers of `zifetar_config(z, layers)`: all three in every four layers, each with a routed feed-forward."""
+    kinds = ["parallel", "channel_delta", "retention", "parallel"]
+    return [kinds[i % 4] for i in range(layers)]
+
+
+def zifetar_sizes(z: dict):
+    """Sizes of the Zifetar layers at the layer sizes `z`: attention as the other designs have it beside a linear attention of
+    half as many heads; a delta rule and retention with as many heads as the attention; 16 gated experts of a quarter of the
+    dense feed-forward's hidden size of which a token uses 4: a token multiplies as much as in the dense gated one.  Chunks as
+    long as the other designs' window."""
+    return dict(lin_heads=z["heads"] // 2, inner=16, experts=16, top=4, expert_ff=z["ff"] // 4, chunk=z["window"])
+
+
+def zifetar_config(z: dict, layers: int):
+    """config.json of a Zifetar model with the layer sizes `z` (see `zifetar_layers`, `zifetar_sizes`)."""
+    n, d = zifetar_sizes(z), z["dim"]
+    out = []
+    for mix in zifetar_layers(layers):
+        if mix == "channel_delta":
+            m = {"heads": z["heads"], "kv_heads": z["heads"], "dim": d, "vdim": d, "conv": 4}
+        elif mix == "retention":
+            m = {"heads": z["heads"], "dim": d, "vdim": d, "rot": {"base": 10000.0, "dims": d},
+                 "decay": [1.0 - 2.0 ** (-5.0 - 7.0 * h / max(1, z["heads"] - 1)) for h in range(z["heads"])]}
+        else:
+            left = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": d, "vdim": d, "scale": d ** -0.5,
+                    "rot": {"base": 500000.0, "dims": d, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+            if n["chunk"]:
+                left["mask"] = {"size": n["chunk"]}
+            m = {"left": left, "right": {"heads": n["lin_heads"], "dim": d, "vdim": d, "tau": 16.0}, "left_scale": 0.7,
+                 "right_scale": 0.7}
+        out.append({"type": mix, "mixer": m, "mlp": {"kind": "moe", "router": {"experts": n["experts"], "top": n["top"]},
+                                                     "expert": {"ff": n["expert_ff"]}}})
+    return {"architecture": "Zifetar", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-6},
+            "embedding": {"scale": 1.0, "bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 1}}, "layers": out}
+
+
+def zifetar_counts(z: dict, layers: int, B: int, C: int, T: int):
+    """(weight elements that a prompt's products multiply a row by, bytes of keys, values and recurrent state that a
+    decode step reads and writes, multiply-adds times two of a prompt's attention and recurrences, weight elements that a
+    decode step of B rows must read) of `zifetar_config(z, layers)`.  A position sees the keys of its own chunk alone; a
+    routed feed-forward multiplies a row by its `top` experts, and a decode step reads the experts that B rows can choose at
+    most.  A recurrence counts as its row-by-row form: two products with the state a row, three by the delta rule."""
+    H, nq, nkv, d = z["width"], z["heads"], z["kv_heads"], z["dim"]
+    n = zifetar_sizes(z)
+    chunk, nl = n["chunk"], n["lin_heads"]
+    w = w_read = kv = att = 0
+    for mix in zifetar_layers(layers):
+        if mix == "channel_delta":
+            m = 4 * nq * d * H + nq * H + 2 * d * H + 2 * nq * d * d
+            kv += B * (nq * d * d + 3 * 3 * nq * d) * 4 * 2
+            att += 6 * T * nq * d * d
+        elif mix == "retention":
+            m = 5 * nq * d * H
+            kv += B * nq * d * d * 4 * 2
+            att += 4 * T * nq * d * d
+        else:
+            m = 2 * nq * d * H + 2 * nkv * d * H + 5 * nl * d * H + n["inner"] * (H + nl * d)
+            seen = ((C - 1) % chunk + 1) if chunk else C
+            kv += B * (seen * nkv * 2 * d * 2 + nl * d * d * 4 * 2)
+            att += 4 * nq * d * sum((p % chunk if chunk else p) + 1 for p in range(T)) + 4 * T * nl * d * d
+        w += m + 3 * H * n["top"] * n["expert_ff"] + n["experts"] * H
+        w_read += m + 3 * H * min(n["experts"], B * n["top"]) * n["expert_ff"] + n["experts"] * H
+    return w, kv, att, w_read
+
+
 def bench_designs(args) -> int:
     """Prefill (one prompt of --prefill-tokens in one step) and decode (--batch sequences at --context
     positions, one token a step through captured graphs) of the designs at equal layer sizes,
@@ -387,6 +453,8 @@ def bench_designs(args) -> int:
             row["giforax"] = measure(giforax_config(z, L), z, counts=giforax_counts(z, L, B, C, T))
         if "zudalorn" in which:
             row["zudalorn"] = measure(zudalorn_config(z, L), z, counts=zudalorn_counts(z, L, B, C, T))
+        if "zifetar" in which:
+            row["zifetar"] = measure(zifetar_config(z, L), z, counts=zifetar_counts(z, L, B, C, T))
         if "sozetar" in which:
             row["sozetar"] = measure(soz, z)
         if "mistral" in which:
@@ -421,10 +489,10 @@ def main() -> int:
     ap.add_argument("--only", choices=["prefill", "decode", "pipes", "designs"], default=None,
                     help="measure one phase only and print its line to stderr (for profiling); pipes: whether a "
                          "SIMD's matrix and vector pipes overlap (ops.measure_pipes); designs: prefill and decode of "
-                         "the Fanitar, Sozetar, Nepisun, Giforax and Zudalorn designs beside the Mistral design at equal layer sizes (--design-sizes, "
+                         "the Fanitar, Sozetar, Nepisun, Giforax, Zudalorn and Zifetar designs beside the Mistral design at equal layer sizes (--design-sizes, "
                          "--layers, --batch, --context, --prefill-tokens apply)")
     ap.add_argument("--design-names", default="fanitar,sozetar,mistral",
-                    help="with --only designs: which designs to run (of fanitar, sozetar, nepisun, giforax, zudalorn, mistral)")
+                    help="with --only designs: which designs to run (of fanitar, sozetar, nepisun, giforax, zudalorn, zifetar, mistral)")
     ap.add_argument("--design-sizes", default="2b,7b,12b",
                     help="with --only designs: which layer sizes to run (of %s)" % ",".join(sorted(DESIGN_SIZES)))
     args = ap.parse_args()

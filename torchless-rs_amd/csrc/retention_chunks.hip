@@ -15,6 +15,7 @@
 // A float that becomes an operand of a product beside the plain rows of q, k and v (the decayed k, the
 // state, the decayed weights of the keys) goes in two bfloat16 terms, x = hi + lo, which carry 16 bits
 // of its mantissa; the sums are float.
+#include "chunks.hpp"
 #include "common.hpp"
 
 namespace tl {
@@ -32,22 +33,6 @@ __device__ __forceinline__ bf16x8 rz8() {
   return z;
 }
 
-// chunk c of the step: its sequence, the step's row it starts at and its rows; false if there is none
-struct Chunk {
-  int b, row0, rows;
-};
-__device__ __forceinline__ bool find_chunk(int c, const int* cu, int B, Chunk& out) {
-  for (int b = 0; b < B; ++b) {
-    const int n = cu[b + 1] - cu[b], chunks = (n + RC - 1) / RC;
-    if (c < chunks) {
-      out = Chunk{b, cu[b] + c * RC, min(RC, n - c * RC)};
-      return true;
-    }
-    c -= chunks;
-  }
-  return false;
-}
-
 // grid (chunks * RC / RC_TILE, H)
 __global__ void __launch_bounds__(256)
 retention_prepare_kernel(const float* __restrict__ proj, int width, int H, int dk, int dv, const int* __restrict__ row_pos,
@@ -57,7 +42,7 @@ retention_prepare_kernel(const float* __restrict__ proj, int width, int H, int d
   extern __shared__ float rc_lds[];                    // [RC_TILE][max(dk, 64) + 1]
   Chunk ch;
   const int c = blockIdx.x / (RC / RC_TILE), t0 = (blockIdx.x % (RC / RC_TILE)) * RC_TILE, h = blockIdx.y, t = threadIdx.x;
-  if (!find_chunk(c, cu, B, ch) || t0 >= ch.rows) return;
+  if (!find_chunk(c, cu, B, RC, ch) || t0 >= ch.rows) return;
   const int rows = min(RC_TILE, ch.rows - t0), n0 = ch.row0 + t0, ld = dk + 1;
   const int half = rot.rotary_dim / 2, units = dk - half;        // a rotated pair, or a channel behind them
   for (int e = t; e < RC_TILE * units; e += 256) {
@@ -136,7 +121,7 @@ retention_states_kernel(const bf16* __restrict__ kt_hi, const bf16* __restrict__
                         int dv, const int* __restrict__ cu, int B, float* __restrict__ kv) {
   Chunk ch;
   const int c = blockIdx.x, h = blockIdx.y, nt = (dv + 63) / 64;
-  if (!find_chunk(c, cu, B, ch)) return;
+  if (!find_chunk(c, cu, B, RC, ch)) return;
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64, l32 = lane % 32, half = lane / 32;
   const int m0 = (blockIdx.z / nt) * 64 + (wave / 2) * 32, n0 = (blockIdx.z % nt) * 64 + (wave % 2) * 32;
   if (m0 >= dk || n0 >= dv) return;
@@ -236,7 +221,7 @@ retention_rows_kernel(const bf16* __restrict__ q, const bf16* __restrict__ k, co
   Chunk ch;
   // the second half of a chunk has the longer way: it goes first
   const int c = blockIdx.x / 2, q0 = (1 - (int)(blockIdx.x % 2)) * RR_BM, h = blockIdx.y;
-  if (!find_chunk(c, cu, B, ch) || q0 >= ch.rows) return;
+  if (!find_chunk(c, cu, B, RC, ch) || q0 >= ch.rows) return;
   const int tid = threadIdx.x, wave = tid / 64, lane = tid % 64, l32 = lane % 32, half = lane / 32;
   const int i = q0 + wave * 32 + l32;                  // this lane's row in the chunk
   const bool ok = i < ch.rows;

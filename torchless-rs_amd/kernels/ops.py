@@ -1530,6 +1530,57 @@ def channel_scan_gated(q, k, v, decay, beta, t: ChannelTerms, state: torch.Tenso
     _channel_scan(q, k, v, decay, beta, t, state, cu_seqlens, slots, None, weight, gate, silu, eps, factor, out)
 
 
+def channel_chunk() -> int:
+    """Rows of a chunk of `channel_chunks`."""
+    return int(lib().tl_channel_chunk())
+
+
+def channel_chunks_serve(dtype: torch.dtype, dk: int, dv: int) -> bool:
+    """Does `channel_chunks` take this dtype and these heads?"""
+    return dtype == torch.bfloat16 and 1 <= dk <= 128 and 1 <= dv <= 256
+
+
+def channel_chunks(proj: torch.Tensor, t: ChannelTerms, z: torch.Tensor, conv_state, state: torch.Tensor, cu_seqlens, slots, chunks: int,
+                   workspace, o: torch.Tensor) -> None:
+    """`channel_rows` and `channel_scan` of a step with many rows, by chunks of `channel_chunk()` rows on the matrix cores: proj
+    as there; z float32 [n, H*dk] = the second step of the decays' projection without its bias; `chunks`: the sequences' new rows
+    in chunks, every sequence's rounded up, added up; `workspace` gives the scratch; o float32 [n, H*dv].  The gate is not made."""
+    n, width = proj.shape
+    B = slots.shape[0]
+    _req_columns(proj, (n, width), "channel_chunks.proj")
+    t.check("channel_chunks")
+    _req(z, "channel_chunks.z", torch.float32, (n, t.H * t.dk))
+    _req_state(state, t.H * t.dk * t.dv, "channel_chunks")
+    if t.taps:
+        _req_state(conv_state, (t.taps - 1) * t.channels, "channel_chunks")
+    _req(cu_seqlens, "channel_chunks.cu_seqlens", torch.int32, (B + 1,))
+    _req(slots, "channel_chunks.slots", torch.int32)
+    _req(o, "channel_chunks.o", torch.float32, (n, t.H * t.dv))
+    if width < t.channels or not channel_chunks_serve(torch.bfloat16, t.dk, t.dv):
+        raise KernelError(f"channel_chunks: heads of {t.dk} and {t.dv} in rows of {width} are not served")
+    delta = t.b_off is not None
+    rec = workspace.get("chunk_rec", (chunks * t.H * int(lib().tl_channel_record(t.dk, int(delta))),), torch.bfloat16)
+    gam = workspace.get("chunk_gam", (chunks * t.H * int(lib().tl_channel_padded(t.dk)),), torch.float32)
+    uf = workspace.get("chunk_u", (chunks * t.H * -(-t.dv // 16) * 1024,), torch.float32)
+    _check(lib().tl_channel_chunks(_p(proj), proj.stride(0), t.G, t.H, t.dk, t.dv, int(t.b_off) if delta else -1, t.taps, _p(t.conv),
+                                   _p(t.bias), _p(t.rate), ctypes.c_float(t.inv_tau), ctypes.c_float(t.qscale),
+                                   ctypes.c_float(-1.0 if t.unit_eps is None else t.unit_eps), _p(z), _p(conv_state),
+                                   ctypes.c_longlong(conv_state.stride(0) if t.taps else 0), _p(state),
+                                   ctypes.c_longlong(state.stride(0)), _p(cu_seqlens), _p(slots), n, B, int(chunks), _p(rec), _p(gam),
+                                   _p(uf), _p(o), _stream()))
+    if t.taps:
+        conv_carry(proj, 0, t.channels, t.taps, conv_state, cu_seqlens, slots)
+
+
+def split_columns(x: torch.Tensor, pad: int, out: torch.Tensor) -> None:
+    """x float32 [n, cols] (rows may be strided) as two bfloat16 terms, x = hi + lo, side by side: out bfloat16 [n, 2 * pad] =
+    [hi | zeros | lo | zeros].  Times [W | W] it gives the product of 16 bits of x's mantissa."""
+    n, cols = x.shape
+    _req_columns(x, (n, cols), "split_columns.x")
+    _req(out, "split_columns.out", torch.bfloat16, (n, 2 * pad))
+    _check(lib().tl_split_columns(_p(x), x.stride(0), cols, int(pad), n, _p(out), _stream()))
+
+
 def take_tokens(src: torch.Tensor, idx: torch.Tensor, vocab: int, tokens: torch.Tensor) -> None:
     """tokens[j] = src[idx[j]] (int32, on the device); ids outside [0, vocab) become 0."""
     n = tokens.shape[0]

@@ -21,8 +21,12 @@ w being one head's weight that all heads share.  The terms are constructor param
 
 The inner sizes of the two-step projections are the tensors' own (`inner` is what a random model
 gets).  What a sequence keeps (`StateRequest`) is of fixed size whatever its length: the convolution's
-last inputs and the states, all float32; nothing per position.  Everything between the two
-products of the mixer is float32 in both dtypes; in bfloat16 the gated result is rounded once.
+last inputs and the states, all float32; nothing per position.
+
+Single tokens, short portions and the 32-bit path go row by row with everything between the two
+products of the mixer in float32 (`ops.channel_rows`, `ops.channel_scan`); longer bfloat16 steps go by chunks of
+rows on the matrix cores (`ops.channel_chunks`), the second steps of the projections as library products of
+their inner rows in two bfloat16 terms.  In bfloat16 the gated result is rounded once.
 """
 from __future__ import annotations
 
@@ -34,7 +38,30 @@ from ..cache.cache import StateRequest
 from ..kernels import ops
 from ..weights.binding import WeightSpec
 from .base import register_part
+from .linear import Linear
 from .projected import ProjectedMixer, same_dtype, stacked
+
+
+CHUNKS_FROM = 32             # a bfloat16 step whose longest sequence brings this many rows goes by chunks
+INNER_STEP = 64              # inner rows are padded to this many channels for the products by their second matrices
+
+
+class SecondStep:
+    """The second matrix [N, rank] of a two-step projection, for rows kept in float: the inner row in two bfloat16 terms
+    [hi | lo] times [W | W]."""
+
+    def __init__(self, weight: torch.Tensor):
+        rank = weight.shape[1]
+        self.pad = -(-rank // INNER_STEP) * INNER_STEP
+        w = torch.zeros((weight.shape[0], 2 * self.pad), dtype=weight.dtype, device=weight.device)
+        w[:, :rank] = weight
+        w[:, self.pad:self.pad + rank] = weight
+        self.w = Linear(w, tiled=False)
+
+    def __call__(self, ctx, inner: torch.Tensor, out: torch.Tensor, name: str) -> None:
+        terms = ctx.workspace.get(name, (inner.shape[0], 2 * self.pad), torch.bfloat16)
+        ops.split_columns(inner, self.pad, terms)
+        self.w(terms, out)
 
 
 class ChannelLinearMixer(ProjectedMixer):
@@ -71,7 +98,13 @@ class ChannelLinearMixer(ProjectedMixer):
         # the states start on a whole vector behind the convolution's rows
         self.conv_elems = -(-max(self.taps - 1, 0) * self.channels // 4) * 4
         self.state_elems = -(-self.heads_n * self.dk * self.dv // 4) * 4
-        self.terms = self.norm_w = None
+        self.terms = self.norm_w = self.decay_step = self.gate_step = None
+
+    def may_capture(self, n_rows: int) -> bool:
+        return super().may_capture(n_rows) and self._steps_capture(n_rows)
+
+    def _steps_capture(self, n_rows: int) -> bool:
+        return all(s.w.own_kernels(n_rows) for s in (self.decay_step, self.gate_step) if s is not None)
 
     def state_request(self):
         return StateRequest((self.conv_elems + self.state_elems,), torch.float32)
@@ -124,6 +157,11 @@ class ChannelLinearMixer(ProjectedMixer):
         second = [m.contiguous() for m in same_dtype([t("decay_out")] + ([t("gate_out")] if two_step else []))]
         self.gate_off = off.get("gate")
         self.norm_w = f32("norm")
+        self.decay_step = self.gate_step = None
+        if ops.channel_chunks_serve(compute_dtype, self.dk, self.dv) and second[0].dtype == torch.bfloat16:
+            self.decay_step = SecondStep(second[0])
+            if two_step:
+                self.gate_step = SecondStep(second[1])
         self.terms = ops.ChannelTerms(
             self.G, self.heads_n, self.dk, self.dv, off["decay_in"], second[0], f32("decay_bias"), off.get("beta"),
             off.get("gate_in"), second[1] if two_step else None,
@@ -138,10 +176,22 @@ class ChannelLinearMixer(ProjectedMixer):
         f32 = torch.float32
         Q, K, V = self.G * self.dk, self.heads_n * self.dk, self.heads_n * self.dv
         conv_state, state = run.state[:, :self.conv_elems], run.state[:, self.conv_elems:]
+        two_step = self.gate == "logistic"
+        if ctx.max_new >= CHUNKS_FROM and self.decay_step is not None:
+            z = ws.get("clin_decay", (n, K), f32)
+            self.decay_step(ctx, proj[:, t.a_off:t.a_off + t.a2.shape[1]], z, "clin_inner")
+            gate = proj[:, self.gate_off:self.gate_off + V] if not two_step else ws.get("clin_gate", (n, V), f32)
+            if two_step:
+                self.gate_step(ctx, proj[:, t.g_off:t.g_off + t.g2.shape[1]], gate, "clin_inner")
+            o = ws.get("clin_o", (n, V), f32)
+            C = ops.channel_chunk()
+            chunks = int(sum(-(-int(r) // C) for r in ctx.host["n_new"]))
+            ops.channel_chunks(proj, t, z, conv_state, state, ctx.cu_seqlens, ctx.slots, chunks, ws, o)
+            ops.heads_norm_gate(o, gate, self.heads_n, self.eps, out, weight=self.norm_w, silu=not two_step, factor=self.factor)
+            return
         q, k, v = ws.get("clin_q", (n, Q), f32), ws.get("clin_k", (n, Q), f32), ws.get("clin_v", (n, V), f32)
         decay = ws.get("clin_decay", (n, K), f32)
         beta = ws.get("clin_beta", (n, self.heads_n), f32) if self.delta else None
-        two_step = self.gate == "logistic"
         gate = ws.get("clin_gate", (n, V), f32) if two_step else proj[:, self.gate_off:self.gate_off + V]
         ops.channel_rows(proj, t, conv_state, ctx.row_seq, ctx.cu_seqlens, ctx.slots, ctx.all_single, q, k, v, decay, beta,
                          gate if two_step else None)

@@ -102,6 +102,9 @@ class ParallelMixer(ProjectedMixer):
     def state_request(self):
         return self._asked("state_request")
 
+    def may_capture(self, n_rows: int) -> bool:
+        return super().may_capture(n_rows) and all(s._steps_capture(n_rows) for s in self.sides if hasattr(s, "_steps_capture"))
+
     def prefers_eager(self, n_new, len_before, device) -> bool:
         return any(s.prefers_eager(n_new, len_before, device) for s in self.sides)
 
