@@ -8,19 +8,21 @@
 //   U = V' - W S ,   o = (D q) S + B U ,   S <- D_last S + (D_last/D k)^T U
 //
 // (the delta rule written for a chunk at once, as in Yang et al., Parallelizing Linear Transformers with
-// the Delta Rule over Sequence Length).  Two kernels:
+// the Delta Rule over Sequence Length).  Three kernels:
 //
 //   local  one workgroup a chunk and head: convolution, unit norms and decays of its rows, A and B, the solution of
-//          the triangular system by blocks of 16 rows, and every operand of the second kernel in the order in which a
+//          the triangular system by blocks of 16 rows, and every operand of the other kernels in the order in which a
 //          wave's lanes take it
-//   carry  one wave 16 columns of a head's state, through the chunks of a sequence in their order, with the state in
-//          its registers in float: a product's result is the next one's operand without leaving them
+//   carry  one workgroup 16 columns of a head's state, through the chunks of a sequence in their order, with the state in
+//          registers in float.  It leaves the state before every chunk and U, as operands
+//   rows   one workgroup a chunk and head: o, the norm over the head and the gate
 //
 // Decays are kept as logarithms (base 2) summed inside blocks of 16 rows, with the blocks' sums beside them: every
-// factor D_i/D_j with j <= i is then 2 to a sum of numbers that are none above 0, whatever the decays; inside a block
-// of 16 rows A and B are summed in float without the matrix cores.  A float that becomes an operand goes in two
-// bfloat16 terms, x = hi + lo (16 bits of its mantissa), and products of two such in three products; only the operands
-// that nothing but a row's own result depends on (D q and B) are rounded to one.  Sums are float.
+// factor D_i/D_j with i and j in different blocks is then a product of two powers of 2 whose exponents are sums of
+// numbers that are none above 0, whatever the decays.  Inside a block the second power has an exponent above 0; a
+// block in which some channel decays by more than 2^-STEEP in all is summed in float pair by pair instead.  A float that becomes an
+// operand goes in two bfloat16 terms, x = hi + lo (16 bits of its mantissa), and products of two such in three products;
+// only operands that nothing but a row's own result depends on (D q and B) are rounded to one.  Sums are float.
 #include "channel_linear.hpp"
 #include "chunks.hpp"
 
@@ -30,6 +32,7 @@ constexpr int CC = 64;               // rows of a chunk
 constexpr int CC_MAX_DK = 128;
 constexpr int FRAG = 512;            // elements of an operand of 16 x 32, lane by lane
 constexpr float LOG2E = 1.4426950408889634f;
+constexpr float STEEP = 60.f;
 
 __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
@@ -69,48 +72,100 @@ struct ChunkArgs {
   int B;
 };
 
-// 16 rows n0 .. of one channel (column c of proj), through the convolution if there is one; rows behind `rows` are zeros
-template <int ROWS>
-__device__ __forceinline__ void channel_run(const ChunkArgs& a, const ChannelTerms& t, int C, int n0, int seq_i0, int rows, const float* st, int c,
-                                            float* out) {
-  float cur[ROWS];
-  const float* p = a.proj + (size_t)n0 * a.width + c;
+__device__ __forceinline__ float rcp_(float x) { return __builtin_amdgcn_rcpf(x); }
+__device__ __forceinline__ float quick_silu(float a) { return a * rcp_(1.f + ex2(-a * LOG2E)); }
+// log2 of a decay (see cl_log_decay) through the exponent and logarithm instructions; log(1 + x) of a small x by its series
+__device__ __forceinline__ float quick_softplus(float a) {
+  const float x = ex2(-fabsf(a) * LOG2E);
+  const float l = x < 0.01f ? x * (1.f - x * (0.5f - x * 0.33333333f)) : __builtin_amdgcn_logf(1.f + x) * 0.69314718f;
+  return fmaxf(a, 0.f) + l;
+}
+__device__ __forceinline__ float log2_decay(float z, bool rated, float rate, float inv_tau) {
+  return (rated ? rate * quick_softplus(z) : -quick_softplus(-z) * inv_tau) * LOG2E;
+}
+
+// ROWS rows n0 .. of one channel (column c of proj) with the rows that a convolution of at most WIN taps looks back to; rows
+// behind `rows` are zeros
+template <int ROWS, int WIN> struct ChannelRun {
+  float cur[ROWS], win[WIN - 1], w[WIN];
+  __device__ __forceinline__ void load(const ChunkArgs& a, const ChannelTerms& t, int C, int n0, int seq_i0, int rows, const float* st, int c) {
+    const float* p = a.proj + (size_t)n0 * a.width + c;
 #pragma unroll
-  for (int r = 0; r < ROWS; ++r) cur[r] = r < rows ? p[(size_t)r * a.width] : 0.f;
-  if (!t.taps) {
+    for (int r = 0; r < ROWS; ++r) cur[r] = r < rows ? p[(size_t)r * a.width] : 0.f;
+    if (!t.taps) return;
 #pragma unroll
-    for (int r = 0; r < ROWS; ++r) out[r] = cur[r];
-    return;
-  }
-  float w[CL_MAX_TAPS], win[CL_MAX_TAPS];              // right-aligned: the last is the present row's
-#pragma unroll
-  for (int j = 0; j < CL_MAX_TAPS; ++j) {
-    const int back = CL_MAX_TAPS - 1 - j;
-    w[j] = back < t.taps ? t.conv_w[(size_t)c * t.taps + t.taps - 1 - back] : 0.f;
-    win[j] = 0.f;
-    if (back > 0 && back < t.taps) {
+    for (int j = 0; j < WIN; ++j) {                    // right-aligned: the last is the present row's
+      const int back = WIN - 1 - j;
+      w[j] = back < t.taps ? t.conv_w[(size_t)c * t.taps + t.taps - 1 - back] : 0.f;
+      if (back == 0) continue;
       const int src = seq_i0 - back;
-      win[j] = src >= 0 ? p[-(ptrdiff_t)back * a.width] : st[(size_t)(t.taps - 1 + src) * C + c];
+      win[j] = 0.f;
+      if (back < t.taps) win[j] = src >= 0 ? p[-(ptrdiff_t)back * a.width] : st[(size_t)(t.taps - 1 + src) * C + c];
     }
   }
+  __device__ __forceinline__ void apply(const ChannelTerms& t, int rows) {
+    if (!t.taps) return;
 #pragma unroll
-  for (int r = 0; r < ROWS; ++r) {
-    win[CL_MAX_TAPS - 1] = cur[r];
-    float acc = 0.f;
+    for (int r = ROWS - 1; r >= 0; --r) {              // (from the last row up: earlier inputs are still as they were)
+      float acc = w[WIN - 1] * cur[r];
 #pragma unroll
-    for (int j = 0; j < CL_MAX_TAPS; ++j) acc = fmaf(w[j], win[j], acc);
-    out[r] = r < rows ? cl_silu(acc) : 0.f;
+      for (int back = 1; back < WIN; ++back) acc = fmaf(w[WIN - 1 - back], r >= back ? cur[r >= back ? r - back : 0] : win[r >= back ? 0 : WIN - 1 + r - back], acc);
+      cur[r] = r < rows ? quick_silu(acc) : 0.f;
+    }
+  }
+};
+
+template <int DK> constexpr size_t local_lds() {
+  return sizeof(float) * (3 * CC * (DK + 4) + 2 * CC * (CC + 4) + 4 * DK + CC + 4 * 16 * 20 + DK / 16);
+}
+
+// (I + M) X = X' by blocks of 16 rows for TILES tiles of 16 columns (a lane holds rows 16 I + 4g .. of column m): M below the
+// diagonal's blocks, T the inverses of those
+template <int TILES>
+__device__ __forceinline__ void solve_tiles(f32x4 (&x)[2][4], const float* Ms, int MLD, const float* Ti, int m, int g) {
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  bf16x8 ph[TILES][2], pl[TILES][2];                   // solved blocks 0, 1 and 2, 3 as operands
 #pragma unroll
-    for (int j = 0; j + 1 < CL_MAX_TAPS; ++j) win[j] = win[j + 1];
+  for (int I = 0; I < 4; ++I) {
+#pragma unroll
+    for (int p = 0; p < 2; ++p) {
+      if (2 * p >= I) continue;
+      float mm[8];
+      const f32x4 m0 = ld4(Ms + (16 * I + m) * MLD + 32 * p + 4 * g);
+      f32x4 m1 = zero;
+      if (2 * p + 1 < I) m1 = ld4(Ms + (16 * I + m) * MLD + 32 * p + 16 + 4 * g);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        mm[e] = -m0[e];
+        mm[4 + e] = -m1[e];
+      }
+      bf16x8 mh, ml;
+      split8(mm, mh, ml);
+#pragma unroll
+      for (int k = 0; k < TILES; ++k) {
+        x[k][I] = mfma16(mh, ph[k][p], x[k][I]);
+        x[k][I] = mfma16(mh, pl[k][p], x[k][I]);
+        x[k][I] = mfma16(ml, ph[k][p], x[k][I]);
+      }
+    }
+    bf16x8 th, tl;
+    split_tiles(ld4(Ti + (I * 16 + m) * 20 + 4 * g), zero, th, tl);
+#pragma unroll
+    for (int k = 0; k < TILES; ++k) {
+      bf16x8 rh, rl;
+      split_tiles(x[k][I], zero, rh, rl);
+      f32x4 y = mfma16(th, rh, zero);
+      y = mfma16(th, rl, y);
+      x[k][I] = mfma16(tl, rh, y);
+      if (I == 0) split_tiles(x[k][0], zero, ph[k][0], pl[k][0]);
+      if (I == 1) split_tiles(x[k][0], x[k][1], ph[k][0], pl[k][0]);
+      if (I == 2) split_tiles(x[k][2], zero, ph[k][1], pl[k][1]);
+    }
   }
 }
 
-template <int DK> constexpr size_t local_lds() {
-  return sizeof(float) * (3 * CC * (DK + 4) + 2 * CC * (CC + 4) + 4 * DK + CC + 4 * 16 * 20);
-}
-
-// grid (chunks, H), 4 * DK threads
-template <int DK, bool DELTA>
+// grid (chunks, H), 4 * DK threads; convolutions of at most WIN taps
+template <int DK, bool DELTA, int WIN>
 __global__ void __launch_bounds__(4 * DK)
 channel_local_kernel(ChunkArgs a, ChannelTerms t, bf16* __restrict__ rec, float* __restrict__ gam, float* __restrict__ uf, int nct) {
   using R = Record<DK, DELTA>;
@@ -124,6 +179,7 @@ channel_local_kernel(ChunkArgs a, ChannelTerms t, bf16* __restrict__ rec, float*
   float* tot = Bs + CC * MLD;            // [4][DK]: a block's sum
   float* bt = tot + 4 * DK;              // [CC]
   float* Ti = bt + CC;                   // [4][16][20]: inverses of the blocks on the diagonal
+  int* steep = reinterpret_cast<int*>(Ti + 4 * 16 * 20);      // [NW]: the wave's channels of its block
   Chunk ch;
   const int c = blockIdx.x, h = blockIdx.y;
   if (!find_chunk(c, a.cu, a.B, CC, ch)) return;
@@ -131,29 +187,37 @@ channel_local_kernel(ChunkArgs a, ChannelTerms t, bf16* __restrict__ rec, float*
   const int kh = h / (t.H / t.G), Q = t.G * t.dk, C = 2 * Q + t.H * t.dv;
   const int seq0 = ch.row0 - a.cu[ch.b];             // the chunk's first row counted from the step's first of the sequence
   const float* st = t.taps ? a.conv_state + (long long)a.slots[ch.b] * a.stride : nullptr;
+  ChannelRun<4, WIN> vr[4];                          // this wave's first tile of values: rows 16 I + 4g .. of column 16 wave + m
   {
     const int d = tid % DK, i0 = (tid / DK) * 16;
-    float x[16];
-    const bool in = d < t.dk;
-    const int rows = in ? ch.rows - i0 : 0, n0 = ch.row0 + i0;
-    if (rows > 0) channel_run<16>(a, t, C, n0, seq0 + i0, rows, st, kh * t.dk + d, x);
+    const int rows = d < t.dk ? ch.rows - i0 : 0, n0 = ch.row0 + i0;
+    ChannelRun<16, WIN> xq, xk;
+    float z[16];
 #pragma unroll
-    for (int r = 0; r < 16; ++r) qs[(i0 + r) * LD + d] = rows > 0 ? x[r] : 0.f;
-    if (rows > 0) channel_run<16>(a, t, C, n0, seq0 + i0, rows, st, Q + kh * t.dk + d, x);
+    for (int r = 0; r < 16; ++r) xq.cur[r] = xk.cur[r] = z[r] = 0.f;
+    float rate = 0.f, bias = 0.f;
+    if (rows > 0) {
+      xq.load(a, t, C, n0, seq0 + i0, rows, st, kh * t.dk + d);
+      xk.load(a, t, C, n0, seq0 + i0, rows, st, Q + kh * t.dk + d);
+      const float* zp = a.z + (size_t)n0 * t.H * t.dk + h * t.dk + d;
 #pragma unroll
-    for (int r = 0; r < 16; ++r) ks[(i0 + r) * LD + d] = rows > 0 ? x[r] : 0.f;
-    const float rate = t.rate ? -expf(t.rate[h]) : 0.f;
-    const float bias = in && t.bias ? t.bias[h * t.dk + d] : 0.f;
-    const float* zp = a.z + (size_t)n0 * t.H * t.dk + h * t.dk + d;
-#pragma unroll
-    for (int r = 0; r < 16; ++r) x[r] = r < rows ? zp[(size_t)r * t.H * t.dk] : 0.f;
+      for (int r = 0; r < 16; ++r) z[r] = r < rows ? zp[(size_t)r * t.H * t.dk] : 0.f;
+      if (t.rate) rate = -expf(t.rate[h]);
+      if (t.bias) bias = t.bias[h * t.dk + d];
+      xq.apply(t, rows);
+      xk.apply(t, rows);
+    }
     float sum = 0.f;
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
-      if (r < rows) sum += cl_log_decay(x[r] + bias, t.rate != nullptr, rate, t.inv_tau) * LOG2E;
+      qs[(i0 + r) * LD + d] = xq.cur[r];
+      ks[(i0 + r) * LD + d] = xk.cur[r];
+      if (r < rows) sum += log2_decay(z[r] + bias, t.rate != nullptr, rate, t.inv_tau);
       ls[(i0 + r) * LD + d] = sum;
     }
     tot[(tid / DK) * DK + d] = sum;
+    const bool any = __any(sum < -STEEP);
+    if (lane == 0) steep[wave] = any;
     if (DELTA && tid < CC)
       bt[tid] = tid < ch.rows ? cl_sigmoid(a.proj[(size_t)(ch.row0 + tid) * a.width + t.b_off + h]) : 0.f;
   }
@@ -194,65 +258,78 @@ channel_local_kernel(ChunkArgs a, ChannelTerms t, bf16* __restrict__ rec, float*
       *reinterpret_cast<f32x4*>(ks + i * LD + e0 + 4 * e) = xk[e];
     }
   }
+  const int vcol = 16 * wave + m;
+#pragma unroll
+  for (int I = 0; I < 4; ++I) {                        // (fetched now, read behind the products below)
+    const int i0 = 16 * I + 4 * g;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) vr[I].cur[r] = 0.f;
+    if (vcol < t.dv && i0 < ch.rows) vr[I].load(a, t, C, ch.row0 + i0, seq0 + i0, ch.rows - i0, st, a.v_off + h * t.dv + vcol);
+  }
   __syncthreads();
 
-  // A (role 0) and B (role 1): blocks on the diagonal in float, those below it on the matrix cores
-  for (int task = (DELTA ? 0 : 4) + wave; task < 8; task += NW) {
-    const int role = task / 4, w4 = task % 4;
-    const float* rs = role ? qs : ks;
-    float* out = role ? Bs : Ms;
-    {
-      const int i = 16 * w4 + m, j0 = 16 * w4 + 4 * g;
-      float acc[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-      for (int d = 0; d < DK; d += 4) {
-        const f32x4 x = ld4(rs + i * LD + d), li = ld4(ls + i * LD + d);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) {
-          const f32x4 y = ld4(ks + (j0 + j) * LD + d), lj = ld4(ls + (j0 + j) * LD + d);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) acc[j] = fmaf(x[e] * y[e], ex2(li[e] - lj[e]), acc[j]);
-        }
-      }
-      const float f = role ? 1.f : bt[i];
-      f32x4 r;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) r[j] = j0 + j < i + role ? acc[j] * f : 0.f;      // (nothing of what lies above is read)
-      *reinterpret_cast<f32x4*>(out + i * MLD + j0) = r;
-    }
-    for (int pair = 0; pair < 2; ++pair) {
-      // wave 0: (3, 0); 1: (3, 1); 2: (3, 2), (1, 0); 3: (2, 0), (2, 1)
-      if (pair == 1 && w4 < 2) break;
-      const int I = w4 == 3 ? 2 : (w4 == 2 && pair ? 1 : 3), J = w4 == 3 ? pair : (w4 == 2 && pair ? 0 : w4);
-      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  // A and B by blocks of 16 x 16
+  for (int p = wave; p < 10; p += NW) {
+    // pairs (3, 0) .. (3, 3), (2, 0) .. (2, 2), (1, 0), (1, 1), (0, 0)
+    const int I = p < 4 ? 3 : (p < 7 ? 2 : (p < 9 ? 1 : 0)), J = p < 4 ? p : (p < 7 ? p - 4 : (p < 9 ? p - 7 : 0));
+    bool exact = false;
+    if (I == J)
+      for (int w = 0; w < DK / WAVE; ++w) exact |= steep[I * (DK / WAVE) + w] != 0;
+    f32x4 aa = {0.f, 0.f, 0.f, 0.f}, ab = aa;          // rows 16 I + 4g .., column 16 J + m
+    if (!exact) {
 #pragma unroll
       for (int s = 0; s < KS; ++s) {
         const int d = 32 * s + 8 * g;
-        float x[8], y[8];
+        float x[8], q[8], y[8];
 #pragma unroll
         for (int q4 = 0; q4 < 2; ++q4) {
-          const f32x4 xr = ld4(rs + (16 * I + m) * LD + d + 4 * q4), li = ld4(ls + (16 * I + m) * LD + d + 4 * q4);
-          const f32x4 yr = ld4(ks + (16 * J + m) * LD + d + 4 * q4), lj = ld4(ls + (16 * J + m) * LD + d + 4 * q4);
-          f32x4 between = ld4(tot + J * DK + d + 4 * q4) - lj;
-          for (int M = J + 1; M < I; ++M) between += ld4(tot + M * DK + d + 4 * q4);
+          const f32x4 li = ld4(ls + (16 * I + m) * LD + d + 4 * q4), lj = ld4(ls + (16 * J + m) * LD + d + 4 * q4);
+          const f32x4 xr = ld4(ks + (16 * I + m) * LD + d + 4 * q4), qr = ld4(qs + (16 * I + m) * LD + d + 4 * q4);
+          const f32x4 yr = ld4(ks + (16 * J + m) * LD + d + 4 * q4);
+          f32x4 between = -lj;
+          for (int M = J; M < I; ++M) between += ld4(tot + M * DK + d + 4 * q4);
 #pragma unroll
           for (int e = 0; e < 4; ++e) {
-            x[4 * q4 + e] = xr[e] * ex2(li[e]);
+            const float f = ex2(li[e]);
+            x[4 * q4 + e] = xr[e] * f;
+            q[4 * q4 + e] = qr[e] * f;
             y[4 * q4 + e] = yr[e] * ex2(between[e]);
           }
         }
         bf16x8 xh, xl, yh, yl;
-        split8(x, xh, xl);
         split8(y, yh, yl);
-        acc = mfma16(xh, yh, acc);
-        acc = mfma16(xh, yl, acc);
-        acc = mfma16(xl, yh, acc);
+        if constexpr (DELTA) {
+          split8(x, xh, xl);
+          aa = mfma16(xh, yh, aa);
+          aa = mfma16(xh, yl, aa);
+          aa = mfma16(xl, yh, aa);
+        }
+        split8(q, xh, xl);
+        ab = mfma16(xh, yh, ab);
+        ab = mfma16(xh, yl, ab);
+        ab = mfma16(xl, yh, ab);
       }
+    } else {                                           // pair by pair: this lane's four rows against its column
+      for (int d = 0; d < DK; d += 4) {
+        const f32x4 y = ld4(ks + (16 * J + m) * LD + d), lj = ld4(ls + (16 * J + m) * LD + d);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int i = 16 * I + 4 * g + r;
-        out[i * MLD + 16 * J + m] = acc[r] * (role ? 1.f : bt[i]);
+        for (int r = 0; r < 4; ++r) {
+          const int i = 16 * I + 4 * g + r;
+          const f32x4 q = ld4(qs + i * LD + d), x = ld4(ks + i * LD + d), li = ld4(ls + i * LD + d);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const float f = y[e] * ex2(fminf(li[e] - lj[e], 0.f));      // (above 0 only for j > i, which is dropped)
+            if constexpr (DELTA) aa[r] = fmaf(x[e], f, aa[r]);
+            ab[r] = fmaf(q[e], f, ab[r]);
+          }
+        }
       }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int i = 16 * I + 4 * g + r, j = 16 * J + m;
+      if constexpr (DELTA) Ms[i * MLD + j] = j < i ? aa[r] * bt[i] : 0.f;
+      Bs[i * MLD + j] = j <= i ? ab[r] : 0.f;
     }
   }
   __syncthreads();
@@ -272,7 +349,7 @@ channel_local_kernel(ChunkArgs a, ChannelTerms t, bf16* __restrict__ rec, float*
       Ti[(wave * 16 + i) * 20 + lane] = x[i];
     }
   }
-  bf16* mine = rec + ((size_t)c * t.H + h) * R::FRAGS * FRAG;
+  bf16* mine = rec + ((size_t)h * gridDim.x + c) * R::FRAGS * FRAG;
   // operands: lane (m, g) of a FRAG holds row m and the eight columns 4g .. 4g+3, 16 + 4g .. 16 + 4g+3 of its 32
   for (int f = wave; f < 4 * KS; f += NW) {            // D q
     const int mt = f / KS, s = f % KS, i = 16 * mt + m;
@@ -320,84 +397,58 @@ channel_local_kernel(ChunkArgs a, ChannelTerms t, bf16* __restrict__ rec, float*
     }
     *reinterpret_cast<bf16x8*>(mine + (size_t)(R::B + f) * FRAG + lane * 8) = v;
   }
-  if (tid < DK) gam[((size_t)c * t.H + h) * DK + tid] = ex2(tot[tid] + tot[DK + tid] + tot[2 * DK + tid] + tot[3 * DK + tid]);
+  if (tid < DK) gam[((size_t)h * gridDim.x + c) * DK + tid] = ex2(tot[tid] + tot[DK + tid] + tot[2 * DK + tid] + tot[3 * DK + tid]);
   __syncthreads();                                     // q has been read: its place takes W
 
   bf16* w_hi = reinterpret_cast<bf16*>(qs);            // [CC][LD]
   bf16* w_lo = w_hi + CC * LD;
-  for (int ct = (DELTA ? 0 : DK / 16) + wave; ct < DK / 16 + nct; ct += NW) {
-    const bool is_w = ct < DK / 16;
-    f32x4 x[4];                                        // rows 16 I + 4 g .. of column m
+  for (int ct = wave; ct == wave || ct < nct; ct += NW) {        // tile ct of the values and, the first time round, of W
+    f32x4 x[2][4];                                     // rows 16 I + 4 g .. of column m
 #pragma unroll
     for (int I = 0; I < 4; ++I) {
-      if (is_w) {
-        const int d = 16 * ct + m;
-        float before = 0.f;
-        for (int M = 0; M < I; ++M) before += tot[M * DK + d];
+      const int i0 = 16 * I + 4 * g;
+      if (ct != wave) {
+        const int col = 16 * ct + m;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int i = 16 * I + 4 * g + r;
-          x[I][r] = bt[i] * ks[i * LD + d] * ex2(before + ls[i * LD + d]);
-        }
-      } else {
-        const int col = 16 * (ct - DK / 16) + m, i0 = 16 * I + 4 * g;
-        float v[4] = {0.f, 0.f, 0.f, 0.f};
-        if (col < t.dv && i0 < ch.rows) channel_run<4>(a, t, C, ch.row0 + i0, seq0 + i0, ch.rows - i0, st, a.v_off + h * t.dv + col, v);
-#pragma unroll
-        for (int r = 0; r < 4; ++r) x[I][r] = DELTA ? bt[i0 + r] * v[r] : v[r];
+        for (int r = 0; r < 4; ++r) vr[I].cur[r] = 0.f;
+        if (col < t.dv && i0 < ch.rows) vr[I].load(a, t, C, ch.row0 + i0, seq0 + i0, ch.rows - i0, st, a.v_off + h * t.dv + col);
       }
+      if (16 * ct + m < t.dv && i0 < ch.rows) vr[I].apply(t, ch.rows - i0);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) x[0][I][r] = DELTA ? bt[i0 + r] * vr[I].cur[r] : vr[I].cur[r];
     }
     if constexpr (DELTA) {
-      bf16x8 ph[2], pl[2];                             // solved blocks 0, 1 and 2, 3 as operands
+      if (ct == wave) {
+        const int d = 16 * ct + m;
+        float before = 0.f;
 #pragma unroll
-      for (int I = 0; I < 4; ++I) {
-        f32x4 acc = x[I];
+        for (int I = 0; I < 4; ++I) {
 #pragma unroll
-        for (int p = 0; p < 2; ++p) {
-          if (2 * p >= I) continue;
-          float mm[8];
-          const f32x4 m0 = ld4(Ms + (16 * I + m) * MLD + 32 * p + 4 * g);
-          f32x4 m1 = {0.f, 0.f, 0.f, 0.f};
-          if (2 * p + 1 < I) m1 = ld4(Ms + (16 * I + m) * MLD + 32 * p + 16 + 4 * g);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            mm[e] = -m0[e];
-            mm[4 + e] = -m1[e];
+          for (int r = 0; r < 4; ++r) {
+            const int i = 16 * I + 4 * g + r;
+            x[1][I][r] = bt[i] * ks[i * LD + d] * ex2(before + ls[i * LD + d]);
           }
-          bf16x8 mh, ml;
-          split8(mm, mh, ml);
-          acc = mfma16(mh, ph[p], acc);
-          acc = mfma16(mh, pl[p], acc);
-          acc = mfma16(ml, ph[p], acc);
+          before += tot[I * DK + d];
         }
-        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-        bf16x8 th, tl, rh, rl;
-        split_tiles(ld4(Ti + (I * 16 + m) * 20 + 4 * g), zero, th, tl);
-        split_tiles(acc, zero, rh, rl);
-        f32x4 y = mfma16(th, rh, zero);
-        y = mfma16(th, rl, y);
-        y = mfma16(tl, rh, y);
-        x[I] = y;
-        if (I == 0) split_tiles(x[0], zero, ph[0], pl[0]);
-        if (I == 1) split_tiles(x[0], x[1], ph[0], pl[0]);
-        if (I == 2) split_tiles(x[2], zero, ph[1], pl[1]);
+        solve_tiles<2>(x, Ms, MLD, Ti, m, g);
+#pragma unroll
+        for (int I = 0; I < 4; ++I)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int at = (16 * I + 4 * g + r) * LD + d;
+            const float v = -x[1][I][r];
+            const bf16 hi = (bf16)v;
+            w_hi[at] = hi;
+            w_lo[at] = (bf16)(v - (float)hi);
+          }
+      } else {
+        solve_tiles<1>(x, Ms, MLD, Ti, m, g);
       }
     }
-    if (is_w) {
+    if (ct < nct) {
+      float* up = uf + (((size_t)h * gridDim.x + c) * nct + ct) * (CC * 16);
 #pragma unroll
-      for (int I = 0; I < 4; ++I)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int at = (16 * I + 4 * g + r) * LD + 16 * ct + m;
-          const float v = -x[I][r];
-          const bf16 hi = (bf16)v;
-          w_hi[at] = hi;
-          w_lo[at] = (bf16)(v - (float)hi);
-        }
-    } else {
-      float* up = uf + (((size_t)c * t.H + h) * nct + ct - DK / 16) * (CC * 16);
-#pragma unroll
-      for (int I = 0; I < 4; ++I) *reinterpret_cast<f32x4*>(up + (I * WAVE + lane) * 4) = x[I];
+      for (int I = 0; I < 4; ++I) *reinterpret_cast<f32x4*>(up + (I * WAVE + lane) * 4) = x[0][I];
     }
   }
   if constexpr (DELTA) {
@@ -417,145 +468,343 @@ channel_local_kernel(ChunkArgs a, ChannelTerms t, bf16* __restrict__ rec, float*
   }
 }
 
-template <int DK, bool DELTA> constexpr size_t carry_lds() { return (size_t)Record<DK, DELTA>::FRAGS * FRAG * sizeof(bf16) + DK * sizeof(float); }
+// what `carry` leaves for a tile of 16 columns of a chunk and head, in FRAGs: the state before the chunk, hi and lo
+// [DK/32][2], and U, hi and lo [2][2]
+template <int DK> struct Carried {
+  static constexpr int U = DK / 16, FRAGS = U + 4;
+};
+constexpr int XCDS = 8;              // parts of the chip with a second-level cache each; workgroups go round them in turn
 
-// grid (H, parts of 64 columns, B), 4 waves
+// 1 KB from memory straight into LDS: lane l's 16 bytes at p to dst + 16 l
+__device__ __forceinline__ void bring(const void* p, void* dst) {
+  __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)p, (__attribute__((address_space(3))) void*)dst, 16, 0, 0);
+}
+template <int N> __device__ __forceinline__ void wait_all_but() {       // until at most N accesses to memory are under way
+  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
+}
+__device__ __forceinline__ void wait_lds() { asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory"); }
+
+// a chunk's place in the ring of `carry`, in KB: W (hi, lo), (D_last/D k)^T (hi, lo), the tile's values, D_last; and, behind the
+// ring, what the waves hand each other: the state (hi, lo) and U (hi, lo) as operands
+template <int DK, bool DELTA> struct Ring {
+  static constexpr int W = 0, K = DELTA ? DK / 4 : 0, U = K + DK / 4, G = U + 4, SLOT = (G + 1) * 1024;
+  static constexpr int SLOTS = SLOT > 48 * 1024 ? 2 : 3;
+  static constexpr int S_OUT = SLOTS * SLOT, U_OUT = S_OUT + DK / 16 * 1024, BYTES = U_OUT + 4 * 1024;
+};
+
+// One workgroup a tile of 16 columns of a head's state; the tiles of a head lie on one part of the chip, where they share
+// what they read.  Wave w keeps rows 32 w .. 32 w + 31 of the state (in its registers, in float) and works out its share of the
+// chunk's 64 rows of U; the waves hand each other the state and U through LDS, a barrier each.  Operands come
+// through a ring in LDS, SLOTS chunks ahead, in two groups a chunk, each issued once the group it replaces has been read.  A
+// wave's accesses complete in their order: it waits until no more are under way than it has issued behind the group (its own
+// share of it; the barrier covers the others'), and behind the last chunk the last one's operands are fetched again, so that
+// the count holds.  grid (XCDS * ceil(H / XCDS) * nct, B), DK / 32 waves
 template <int DK, bool DELTA>
-__global__ void __launch_bounds__(256, 1)
-channel_carry_kernel(const bf16* __restrict__ rec, const float* __restrict__ gam, const float* __restrict__ uf, int nct, int H, int dk, int dv,
-                     float* __restrict__ state, long long stride, const int* __restrict__ cu, const int* __restrict__ slots,
-                     float* __restrict__ o) {
+__global__ void __launch_bounds__(2 * DK)
+channel_carry_kernel(const bf16* __restrict__ rec, const float* __restrict__ gam, const float* __restrict__ uf, int nct, int total, int H, int dk,
+                     int dv, float* __restrict__ state, long long stride, const int* __restrict__ cu, const int* __restrict__ slots,
+                     bf16* __restrict__ su) {
   using R = Record<DK, DELTA>;
-  constexpr int KS = DK / 32, MT = DK / 16, LOADS = R::FRAGS * FRAG * 2 / (256 * 16);
-  extern __shared__ __attribute__((aligned(16))) bf16 cy_lds[];
-  float* gs = reinterpret_cast<float*>(cy_lds + R::FRAGS * FRAG);       // [DK]
-  const int h = blockIdx.x, b = blockIdx.z;
-  const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE, m = lane % 16, g = lane / 16;
-  const int ct = blockIdx.y * 4 + wave, col = 16 * ct + m;
+  using S_ = Carried<DK>;
+  using L = Ring<DK, DELTA>;
+  constexpr int KS = DK / 32, NS = L::SLOTS, RI = 4 / KS;        // RI: blocks of 16 rows of U a wave
+  constexpr int G1 = (DELTA ? 8 : 0) + RI + 1, G2 = 8, BEHIND = (NS - 1) * (G1 + G2);
+  extern __shared__ __attribute__((aligned(1024))) unsigned char ring[];
+  const int idx = blockIdx.x / XCDS, h = blockIdx.x % XCDS + XCDS * (idx / nct), ct = idx % nct, b = blockIdx.y;
+  if (h >= H) return;
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE, m = lane % 16, g = lane / 16, col = 16 * ct + m;
   int first = 0;
   for (int s = 0; s < b; ++s) first += (cu[s + 1] - cu[s] + CC - 1) / CC;
-  const int row0 = cu[b], n = cu[b + 1] - row0, chunks = (n + CC - 1) / CC;
+  const int n = cu[b + 1] - cu[b], chunks = (n + CC - 1) / CC;
   if (chunks == 0) return;
-  const bool active = ct < nct;
-  const bool ok = active && col < dv;
+  const bool ok = col < dv;
   float* S_g = state + (long long)slots[b] * stride + ((size_t)h * dv + (ok ? col : 0)) * dk;
-  f32x4 S[MT];
+  f32x4 S[2];                                          // rows 32 wave + 16 t + 4g .. of column m
 #pragma unroll
-  for (int mt = 0; mt < MT; ++mt)
+  for (int t = 0; t < 2; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int d = 16 * mt + 4 * g + r;
-      S[mt][r] = ok && d < dk ? S_g[d] : 0.f;
+      const int d = 32 * wave + 16 * t + 4 * g + r;
+      S[t][r] = ok && d < dk ? S_g[d] : 0.f;
     }
-  f32x4 stage[LOADS], gst, u0[4], un[4];
-  auto load = [&](int c) {
-    const size_t at = (size_t)(first + c) * H + h;
-    const f32x4* src = reinterpret_cast<const f32x4*>(rec + at * R::FRAGS * FRAG);
+  // group 1 of a chunk: W, the values, D_last; group 2: (D_last/D k)^T.  Every wave its share (D_last: each, the same)
+  auto issue1 = [&](int c) {
+    const size_t at = (size_t)h * total + first + min(c, chunks - 1);
+    unsigned char* slot = ring + (c % NS) * L::SLOT;
+    if constexpr (DELTA) {
+      const bf16* p = rec + (at * R::FRAGS + R::W_HI + 8 * wave) * FRAG + lane * 8;
 #pragma unroll
-    for (int e = 0; e < LOADS; ++e) stage[e] = src[e * 256 + tid];
-    if (tid < DK / 4) gst = ld4(gam + at * DK + 4 * tid);
-    if (active) {
-      const float* up = uf + (at * nct + ct) * (CC * 16);
-#pragma unroll
-      for (int I = 0; I < 4; ++I) un[I] = ld4(up + (I * WAVE + lane) * 4);
+      for (int f = 0; f < 8; ++f) bring(p + f * FRAG, slot + (L::W + 8 * wave + f) * 1024);
     }
+    const float* up = uf + (at * nct + ct) * (CC * 16) + RI * wave * WAVE * 4 + lane * 4;
+#pragma unroll
+    for (int I = 0; I < RI; ++I) bring(up + I * WAVE * 4, slot + (L::U + RI * wave + I) * 1024);
+    bring(gam + at * DK + (lane * 4) % DK, slot + L::G * 1024);
   };
-  auto frag = [&](int f) { return *reinterpret_cast<const bf16x8*>(cy_lds + f * FRAG + lane * 8); };
-  load(0);
-  for (int c = 0; c < chunks; ++c) {
-    __syncthreads();                                   // the chunk before has been worked on
+  auto issue2 = [&](int c) {
+    const size_t at = (size_t)h * total + first + min(c, chunks - 1);
+    const bf16* p = rec + (at * R::FRAGS + R::K_HI + 8 * wave) * FRAG + lane * 8;
+    unsigned char* slot = ring + (c % NS) * L::SLOT;
 #pragma unroll
-    for (int e = 0; e < LOADS; ++e) reinterpret_cast<f32x4*>(cy_lds)[e * 256 + tid] = stage[e];
-    if (tid < DK / 4) *reinterpret_cast<f32x4*>(gs + 4 * tid) = gst;
-#pragma unroll
-    for (int I = 0; I < 4; ++I) u0[I] = un[I];
-    __syncthreads();
-    if (c + 1 < chunks) load(c + 1);
-    if (!active) continue;
-    f32x4 out[4];
-#pragma unroll
-    for (int I = 0; I < 4; ++I) out[I] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int s = 0; s < KS; ++s) {
-      bf16x8 sh, sl;
-      split_tiles(S[2 * s], S[2 * s + 1], sh, sl);
-#pragma unroll
-      for (int I = 0; I < 4; ++I) {
-        if constexpr (DELTA) {
-          const bf16x8 wh = frag(R::W_HI + I * KS + s), wl = frag(R::W_LO + I * KS + s);
-          u0[I] = mfma16(wh, sh, u0[I]);
-          u0[I] = mfma16(wh, sl, u0[I]);
-          u0[I] = mfma16(wl, sh, u0[I]);
-        }
-        const bf16x8 qf = frag(R::Q + I * KS + s);
-        out[I] = mfma16(qf, sh, out[I]);
-        out[I] = mfma16(qf, sl, out[I]);
-      }
-    }
-    bf16x8 uh[2], ul[2];
-    split_tiles(u0[0], u0[1], uh[0], ul[0]);
-    split_tiles(u0[2], u0[3], uh[1], ul[1]);
-#pragma unroll
-    for (int mt = 0; mt < MT; ++mt) {
-      S[mt] *= ld4(gs + 16 * mt + 4 * g);
-#pragma unroll
-      for (int s = 0; s < 2; ++s) {
-        const bf16x8 kh = frag(R::K_HI + 2 * mt + s), kl = frag(R::K_LO + 2 * mt + s);
-        S[mt] = mfma16(kh, uh[s], S[mt]);
-        S[mt] = mfma16(kh, ul[s], S[mt]);
-        S[mt] = mfma16(kl, uh[s], S[mt]);
-      }
-    }
-#pragma unroll
-    for (int I = 0; I < 4; ++I) {
-#pragma unroll
-      for (int s = 0; s < 2; ++s) {
-        if (2 * s > I) continue;                       // (B is zero above the diagonal)
-        const bf16x8 bf = frag(R::B + 2 * I + s);
-        out[I] = mfma16(bf, uh[s], out[I]);
-        out[I] = mfma16(bf, ul[s], out[I]);
-      }
-      if (ok) {
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int i = c * CC + 16 * I + 4 * g + r;
-          if (i < n) o[((size_t)(row0 + i) * H + h) * dv + col] = out[I][r];
-        }
-      }
-    }
+    for (int f = 0; f < 8; ++f) bring(p + f * FRAG, slot + (L::K + 8 * wave + f) * 1024);
+  };
+  for (int c = 0; c < NS; ++c) {
+    issue1(c);
+    if (c + 1 < NS) issue2(c);
   }
+  bf16* sp = su + (((size_t)h * total + first) * nct + ct) * S_::FRAGS * FRAG + lane * 8;
+  const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+  for (int c = 0; c < chunks; ++c) {
+    const unsigned char* slot = ring + (c % NS) * L::SLOT;
+    auto frag = [&](const unsigned char* p) { return *reinterpret_cast<const bf16x8*>(p + lane * 16); };
+    bf16x8 hi, lo;
+    split_tiles(S[0], S[1], hi, lo);                   // this wave's rows of the state as an operand
+    if constexpr (DELTA) {
+      *reinterpret_cast<bf16x8*>(ring + L::S_OUT + (2 * wave) * 1024 + lane * 16) = hi;
+      *reinterpret_cast<bf16x8*>(ring + L::S_OUT + (2 * wave + 1) * 1024 + lane * 16) = lo;
+    }
+    wait_all_but<BEHIND>();
+    wait_lds();
+    __builtin_amdgcn_s_barrier();                      // group 1 and every wave's state are there; the last group 2 has been read
+    issue2(c + NS - 1);
+    *reinterpret_cast<bf16x8*>(sp + (size_t)(2 * wave) * FRAG) = hi;
+    *reinterpret_cast<bf16x8*>(sp + (size_t)(2 * wave + 1) * FRAG) = lo;
+    f32x4 gn[2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) gn[t] = *reinterpret_cast<const f32x4*>(slot + L::G * 1024 + (32 * wave + 16 * t + 4 * g) * 4);
+    f32x4 u[RI], u1[RI], u2[RI];
+#pragma unroll
+    for (int I = 0; I < RI; ++I) {
+      u[I] = *reinterpret_cast<const f32x4*>(slot + (L::U + RI * wave + I) * 1024 + lane * 16);
+      u1[I] = u2[I] = zero;
+    }
+    if constexpr (DELTA) {
+#pragma unroll
+      for (int s = 0; s < KS; ++s) {
+        const bf16x8 sh = frag(ring + L::S_OUT + (2 * s) * 1024), sl = frag(ring + L::S_OUT + (2 * s + 1) * 1024);
+#pragma unroll
+        for (int I = 0; I < RI; ++I) {
+          const int f = (RI * wave + I) * KS + s;
+          const bf16x8 wh = frag(slot + (L::W + f) * 1024), wl = frag(slot + (L::W + 4 * KS + f) * 1024);
+          u[I] = mfma16(wh, sh, u[I]);
+          u1[I] = mfma16(wh, sl, u1[I]);
+          u2[I] = mfma16(wl, sh, u2[I]);
+        }
+      }
+    }
+#pragma unroll
+    for (int I = 0; I < RI; ++I) {                     // this wave's rows of U, half of an operand each
+      const f32x4 x = u[I] + (u1[I] + u2[I]);
+      const int at = RI * wave + I, p = (S_::U + 2 * (at / 2)) * FRAG + (at % 2) * 4, q = L::U_OUT + 2 * (at / 2) * 1024 + (at % 2) * 8;
+      bf16x4 uh, ul;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        uh[r] = (bf16)x[r];
+        ul[r] = (bf16)(x[r] - (float)uh[r]);
+      }
+      *reinterpret_cast<bf16x4*>(ring + q + lane * 16) = uh;
+      *reinterpret_cast<bf16x4*>(ring + q + 1024 + lane * 16) = ul;
+      *reinterpret_cast<bf16x4*>(sp + p) = uh;
+      *reinterpret_cast<bf16x4*>(sp + p + FRAG) = ul;
+    }
+    wait_all_but<BEHIND>();
+    wait_lds();
+    __builtin_amdgcn_s_barrier();                      // group 2 and every wave's U are there; group 1 has been read
+    issue1(c + NS);
+    f32x4 lowS[2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      S[t] *= gn[t];
+      lowS[t] = zero;
+    }
+#pragma unroll
+    for (int s = 0; s < 2; ++s) {
+      const bf16x8 uh = frag(ring + L::U_OUT + (2 * s) * 1024), ul = frag(ring + L::U_OUT + (2 * s + 1) * 1024);
+#pragma unroll
+      for (int t = 0; t < 2; ++t) {
+        const int f = 2 * (2 * wave + t) + s;
+        const bf16x8 kh = frag(slot + (L::K + f) * 1024), kl = frag(slot + (L::K + DK / 8 + f) * 1024);
+        S[t] = mfma16(kh, uh, S[t]);
+        lowS[t] = mfma16(kh, ul, lowS[t]);
+        lowS[t] = mfma16(kl, uh, lowS[t]);
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < 2; ++t) S[t] += lowS[t];
+    sp += (size_t)nct * S_::FRAGS * FRAG;
+  }
+  wait_all_but<0>();                                   // (nothing may arrive in LDS behind the wave's end)
   if (!ok) return;
 #pragma unroll
-  for (int mt = 0; mt < MT; ++mt)
+  for (int t = 0; t < 2; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int d = 16 * mt + 4 * g + r;
-      if (d < dk) S_g[d] = S[mt][r];
+      const int d = 32 * wave + 16 * t + 4 * g + r;
+      if (d < dk) S_g[d] = S[t][r];
     }
 }
 
+struct RowsOut {
+  const float* w;            // [dv] (null: no weight)
+  const float* gate;         // the gate's first column in rows `gate_stride` apart
+  int gate_stride, gate_silu;
+  float eps, factor;
+  bf16* out;                 // rows `out_stride` apart
+  int out_stride;
+};
+constexpr int RW_NT = 512, RW_TILES = 2;      // threads; tiles of 16 columns a wave at most (dv up to 256)
+
+// out = factor * rms(o) * w * gate with o = (D q) S + B U.  grid (chunks, H)
 template <int DK, bool DELTA>
-static int launch_chunks(const ChunkArgs& a, const ChannelTerms& t, int chunks, bf16* rec, float* gam, float* uf, float* state, long long stride,
-                         float* o, hipStream_t st) {
+__global__ void __launch_bounds__(RW_NT)
+channel_out_kernel(const bf16* __restrict__ rec, const bf16* __restrict__ su, int nct, int H, int dv, const int* __restrict__ cu, int B,
+                   RowsOut z) {
+  using R = Record<DK, DELTA>;
+  using S_ = Carried<DK>;
+  constexpr int KS = DK / 32, NW = RW_NT / WAVE;
+  extern __shared__ __attribute__((aligned(16))) unsigned char rw_lds[];
+  const int ld = 16 * nct + 8;
+  bf16* os = reinterpret_cast<bf16*>(rw_lds);                            // [CC][ld]
+  float* sums = reinterpret_cast<float*>(os + CC * ld);                   // [NW][CC]
+  Chunk ch;
+  const int c = blockIdx.x, h = blockIdx.y;
+  if (!find_chunk(c, cu, B, CC, ch)) return;
+  const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE, m = lane % 16, g = lane / 16;
+  const bf16* mine = rec + ((size_t)h * gridDim.x + c) * R::FRAGS * FRAG + lane * 8;
+  const bf16* sp = su + ((size_t)h * gridDim.x + c) * nct * S_::FRAGS * FRAG + lane * 8;
+  auto frag = [&](const bf16* p, int f) { return *reinterpret_cast<const bf16x8*>(p + (size_t)f * FRAG); };
+  f32x4 o[RW_TILES][4], gt[RW_TILES][4];
+  f32x4 ss[4];
+#pragma unroll
+  for (int k = 0; k < RW_TILES; ++k) {                 // the gates, fetched ahead
+    const int col = 16 * (wave + k * NW) + m;
+#pragma unroll
+    for (int I = 0; I < 4; ++I)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 16 * I + 4 * g + r;
+        gt[k][I][r] = col < dv && i < ch.rows ? z.gate[(size_t)(ch.row0 + i) * z.gate_stride + (size_t)h * dv + col] : 0.f;
+      }
+  }
+#pragma unroll
+  for (int I = 0; I < 4; ++I) ss[I] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int k = 0; k < RW_TILES; ++k) {
+    const int ct = wave + k * NW;
+    if (ct >= nct) break;
+    const bf16* tp = sp + (size_t)ct * S_::FRAGS * FRAG;
+#pragma unroll
+    for (int I = 0; I < 4; ++I) o[k][I] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < KS; ++s) {
+      const bf16x8 sh = frag(tp, 2 * s), sl = frag(tp, 2 * s + 1);
+#pragma unroll
+      for (int I = 0; I < 4; ++I) {
+        const bf16x8 q = frag(mine, R::Q + I * KS + s);
+        o[k][I] = mfma16(q, sh, o[k][I]);
+        o[k][I] = mfma16(q, sl, o[k][I]);
+      }
+    }
+#pragma unroll
+    for (int s = 0; s < 2; ++s) {
+      const bf16x8 uh = frag(tp, S_::U + 2 * s), ul = frag(tp, S_::U + 2 * s + 1);
+#pragma unroll
+      for (int I = 2 * s; I < 4; ++I) {                // (B is zero above the diagonal)
+        const bf16x8 bb = frag(mine, R::B + 2 * I + s);
+        o[k][I] = mfma16(bb, uh, o[k][I]);
+        o[k][I] = mfma16(bb, ul, o[k][I]);
+      }
+    }
+#pragma unroll
+    for (int I = 0; I < 4; ++I) ss[I] += o[k][I] * o[k][I];      // (columns behind dv are zeros)
+  }
+#pragma unroll
+  for (int I = 0; I < 4; ++I)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float sum = row16_sum(ss[I][r]);
+      if (m == 0) sums[wave * CC + 16 * I + 4 * g + r] = sum;
+    }
+  __syncthreads();
+#pragma unroll
+  for (int I = 0; I < 4; ++I)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      float sum = 0.f;
+#pragma unroll
+      for (int w = 0; w < NW; ++w) sum += sums[w * CC + 16 * I + 4 * g + r];
+      ss[I][r] = z.factor / sqrtf(sum / (float)dv + z.eps);
+    }
+#pragma unroll
+  for (int k = 0; k < RW_TILES; ++k) {
+    const int ct = wave + k * NW, col = 16 * ct + m;
+    if (ct >= nct) break;
+    if (col >= dv) continue;
+    const float wc = z.w ? z.w[col] : 1.f;
+#pragma unroll
+    for (int I = 0; I < 4; ++I)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 16 * I + 4 * g + r;
+        if (i >= ch.rows) continue;
+        const float a = gt[k][I][r];
+        os[i * ld + col] = (bf16)(o[k][I][r] * ss[I][r] * wc * ((z.gate_silu ? a : 1.f) * rcp_(1.f + ex2(-a * LOG2E))));
+      }
+  }
+  __syncthreads();
+  bf16* out = z.out + (size_t)ch.row0 * z.out_stride + (size_t)h * dv;
+  if (dv % 8 == 0 && z.out_stride % 8 == 0 && (uintptr_t)z.out % 16 == 0) {
+    const int per = dv / 8;
+    for (int e = tid; e < ch.rows * per; e += RW_NT) {
+      const int i = e / per, col = (e % per) * 8;
+      *reinterpret_cast<bf16x8*>(out + (size_t)i * z.out_stride + col) = *reinterpret_cast<const bf16x8*>(os + i * ld + col);
+    }
+  } else {
+    for (int e = tid; e < ch.rows * dv; e += RW_NT) out[(size_t)(e / dv) * z.out_stride + e % dv] = os[(e / dv) * ld + e % dv];
+  }
+}
+
+template <int DK, bool DELTA, int WIN>
+static int launch_local(const ChunkArgs& a, const ChannelTerms& t, int chunks, bf16* rec, float* gam, float* uf, int nct, hipStream_t st) {
   static bool raised = false;
   if (!raised) {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&channel_local_kernel<DK, DELTA>),
-                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)local_lds<DK>());
-    if (e == hipSuccess)
-      e = hipFuncSetAttribute(reinterpret_cast<const void*>(&channel_carry_kernel<DK, DELTA>),
-                              hipFuncAttributeMaxDynamicSharedMemorySize, (int)carry_lds<DK, DELTA>());
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&channel_local_kernel<DK, DELTA, WIN>),
+                                             hipFuncAttributeMaxDynamicSharedMemorySize, (int)local_lds<DK>());
     if (e != hipSuccess) {
-      set_error("channel_chunks: cannot have %zu and %zu bytes of LDS: %s", local_lds<DK>(), carry_lds<DK, DELTA>(), hipGetErrorString(e));
+      set_error("channel_chunks: cannot have %zu bytes of LDS: %s", local_lds<DK>(), hipGetErrorString(e));
       return 2;
     }
     raised = true;
   }
-  const int nct = (t.dv + 15) / 16;
-  channel_local_kernel<DK, DELTA><<<dim3(chunks, t.H), 4 * DK, local_lds<DK>(), st>>>(a, t, rec, gam, uf, nct);
+  channel_local_kernel<DK, DELTA, WIN><<<dim3(chunks, t.H), 4 * DK, local_lds<DK>(), st>>>(a, t, rec, gam, uf, nct);
   TL_LAUNCH_CHECK("channel_local");
-  channel_carry_kernel<DK, DELTA><<<dim3(t.H, (nct + 3) / 4, a.B), 256, carry_lds<DK, DELTA>(), st>>>(rec, gam, uf, nct, t.H, t.dk, t.dv, state,
-                                                                                                 stride, a.cu, a.slots, o);
+  return 0;
+}
+
+template <int DK, bool DELTA>
+static int launch_chunks(const ChunkArgs& a, const ChannelTerms& t, int chunks, bf16* rec, float* gam, float* uf, bf16* su, float* state,
+                         long long stride, const RowsOut& z, hipStream_t st) {
+  const int nct = (t.dv + 15) / 16;
+  const int rc = t.taps <= 4 ? launch_local<DK, DELTA, 4>(a, t, chunks, rec, gam, uf, nct, st)
+                             : launch_local<DK, DELTA, CL_MAX_TAPS>(a, t, chunks, rec, gam, uf, nct, st);
+  if (rc) return rc;
+  constexpr int ring = Ring<DK, DELTA>::BYTES;
+  static bool raised = false;
+  if (!raised) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&channel_carry_kernel<DK, DELTA>),
+                                             hipFuncAttributeMaxDynamicSharedMemorySize, ring);
+    if (e != hipSuccess) {
+      set_error("channel_chunks: cannot have %d bytes of LDS: %s", ring, hipGetErrorString(e));
+      return 2;
+    }
+    raised = true;
+  }
+  channel_carry_kernel<DK, DELTA><<<dim3(XCDS * ((t.H + XCDS - 1) / XCDS) * nct, a.B), 2 * DK, ring, st>>>(rec, gam, uf, nct, chunks, t.H, t.dk,
+                                                                                                        t.dv, state, stride, a.cu, a.slots, su);
   TL_LAUNCH_CHECK("channel_carry");
+  const size_t lds = (size_t)CC * (16 * nct + 8) * sizeof(bf16) + (RW_NT / WAVE) * CC * sizeof(float);
+  channel_out_kernel<DK, DELTA><<<dim3(chunks, t.H), RW_NT, lds, st>>>(rec, su, nct, t.H, t.dv, a.cu, a.B, z);
+  TL_LAUNCH_CHECK("channel_out");
   return 0;
 }
 
@@ -585,6 +834,8 @@ int tl_channel_record(int dk, int delta) {
   return (delta ? Record<128, true>::FRAGS : Record<128, false>::FRAGS) * FRAG;
 }
 int tl_channel_padded(int dk) { return dk <= 64 ? 64 : 128; }
+// bfloat16 elements that `carry` leaves for a tile of 16 columns of a chunk and head
+int tl_channel_carried(int dk) { return (dk <= 64 ? Carried<64>::FRAGS : Carried<128>::FRAGS) * FRAG; }
 
 int tl_split_columns(const float* x, int stride, int cols, int pad, int n, void* out, hipStream_t st) {
   TL_REQUIRE(n >= 0 && cols > 0 && cols <= pad && stride >= cols && x && out, "split_columns: bad arguments n=%d cols=%d pad=%d", n, cols, pad);
@@ -597,12 +848,13 @@ int tl_split_columns(const float* x, int stride, int cols, int pad, int n, void*
 }
 
 // proj [n, width] float = [q | k | v | ..]; z [n, H*dk] float (second step of the decays, without the bias); `chunks`: the step's
-// chunks.  Scratch: rec chunks*H*tl_channel_record, gam chunks*H*tl_channel_padded floats, uf chunks*H*ceil(dv/16)*1024 floats.
-// o float [n, H*dv].
+// chunks.  Scratch: rec chunks*H*tl_channel_record, gam chunks*H*tl_channel_padded floats, uf chunks*H*ceil(dv/16)*1024 floats, su
+// chunks*H*ceil(dv/16)*tl_channel_carried.  out bfloat16 [n, H*dv] = factor * rms(o) * w * (silu or logistic of gate).
 int tl_channel_chunks(const float* proj, int width, int G, int H, int dk, int dv, int b_off, int taps, const float* conv_w, const float* bias,
                       const float* rate, float inv_tau, float qscale, float unit_eps, const float* z, const float* conv_state,
                       long long conv_stride, float* state, long long stride, const int* cu, const int* slots, int n, int B, int chunks,
-                      void* rec, float* gam, float* uf, float* o, hipStream_t st) {
+                      void* rec, float* gam, float* uf, void* su, const float* w, const float* gate, int gate_stride, int gate_silu,
+                      float eps, float factor, void* out, int out_stride, hipStream_t st) {
   TL_REQUIRE(n > 0 && B > 0 && B <= 65535 && G > 0 && H > 0 && H <= 65535 && H % G == 0 && chunks > 0, "channel_chunks: bad sizes n=%d B=%d G=%d H=%d chunks=%d",
              n, B, G, H, chunks);
   TL_REQUIRE(dk > 0 && dk <= CC_MAX_DK && dv > 0 && dv <= CL_MAX_D, "channel_chunks: heads of %d and %d are not served (up to %d and %d)", dk, dv,
@@ -611,18 +863,20 @@ int tl_channel_chunks(const float* proj, int width, int G, int H, int dk, int dv
   TL_REQUIRE(C <= width && b_off + (b_off < 0 ? 0 : H) <= width, "channel_chunks: a row of %d is too short", width);
   TL_REQUIRE(taps >= 0 && taps <= CL_MAX_TAPS && (taps == 0 || (conv_w && conv_state && conv_stride >= (long long)(taps - 1) * C)),
              "channel_chunks: a convolution of %d taps without weights, or a block too small", taps);
-  TL_REQUIRE(proj && z && state && cu && slots && rec && gam && uf && o, "channel_chunks: a buffer is missing");
-  TL_REQUIRE(((uintptr_t)rec | (uintptr_t)gam | (uintptr_t)uf) % 16 == 0, "channel_chunks: a buffer off 16 bytes");
+  TL_REQUIRE(proj && z && state && cu && slots && rec && gam && uf && su && gate && out, "channel_chunks: a buffer is missing");
+  TL_REQUIRE(((uintptr_t)rec | (uintptr_t)gam | (uintptr_t)uf | (uintptr_t)su) % 16 == 0, "channel_chunks: a buffer off 16 bytes");
   TL_REQUIRE(stride >= (long long)H * dk * dv, "channel_chunks: a sequence's block is too small");
+  TL_REQUIRE(gate_stride >= H * dv && out_stride >= H * dv, "channel_chunks: rows of the gate or the result are too short");
   const ChunkArgs a{proj, width, 2 * G * dk, z, conv_state, conv_stride, cu, slots, B};
   const ChannelTerms t{G, H, dk, dv, b_off, 0, 0, 0, 0, taps, conv_w, bias, rate, inv_tau, qscale, unit_eps};
+  const RowsOut r{w, gate, gate_stride, gate_silu, eps, factor, (bf16*)out, out_stride};
   const bool delta = b_off >= 0;
   if (dk <= 64) {
-    if (delta) return launch_chunks<64, true>(a, t, chunks, (bf16*)rec, gam, uf, state, stride, o, st);
-    return launch_chunks<64, false>(a, t, chunks, (bf16*)rec, gam, uf, state, stride, o, st);
+    if (delta) return launch_chunks<64, true>(a, t, chunks, (bf16*)rec, gam, uf, (bf16*)su, state, stride, r, st);
+    return launch_chunks<64, false>(a, t, chunks, (bf16*)rec, gam, uf, (bf16*)su, state, stride, r, st);
   }
-  if (delta) return launch_chunks<128, true>(a, t, chunks, (bf16*)rec, gam, uf, state, stride, o, st);
-  return launch_chunks<128, false>(a, t, chunks, (bf16*)rec, gam, uf, state, stride, o, st);
+  if (delta) return launch_chunks<128, true>(a, t, chunks, (bf16*)rec, gam, uf, (bf16*)su, state, stride, r, st);
+  return launch_chunks<128, false>(a, t, chunks, (bf16*)rec, gam, uf, (bf16*)su, state, stride, r, st);
 }
 
 }  // extern "C"

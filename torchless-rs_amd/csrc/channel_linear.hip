@@ -32,15 +32,6 @@ namespace tl {
 
 constexpr int CL_TB = 4;             // rows of a sequence that the scan stages at a time
 
-// Sum over the 16 lanes of a row of a wave; every lane gets it.
-__device__ __forceinline__ float row16_sum(float v) {
-  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x128, 0xf, 0xf, true));   // row_ror:8
-  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x124, 0xf, 0xf, true));   // row_ror:4
-  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x122, 0xf, 0xf, true));   // row_ror:2
-  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x121, 0xf, 0xf, true));   // row_ror:1
-  return v;
-}
-
 // out[c] (for c of this wave's lanes) = sum_r W2[first + c, r] * a[r]
 template <typename T>
 __device__ __forceinline__ float second_step(const T* __restrict__ w2, size_t row, const float* __restrict__ a, int rank) {

@@ -17,6 +17,15 @@ __device__ __forceinline__ float cl_log_decay(float z, bool rated, float rate, f
   return rated ? rate * cl_softplus(z) : -cl_softplus(-z) * inv_tau;
 }
 
+// Sum over the 16 lanes of a row of a wave; every lane gets it.
+__device__ __forceinline__ float row16_sum(float v) {
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x128, 0xf, 0xf, true));   // row_ror:8
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x124, 0xf, 0xf, true));   // row_ror:4
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x122, 0xf, 0xf, true));   // row_ror:2
+  v += __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x121, 0xf, 0xf, true));   // row_ror:1
+  return v;
+}
+
 struct ChannelTerms {
   int G, H, dk, dv;
   int b_off;                 // beta's column (-1: the plain recurrence)

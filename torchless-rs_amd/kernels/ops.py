@@ -1541,10 +1541,11 @@ def channel_chunks_serve(dtype: torch.dtype, dk: int, dv: int) -> bool:
 
 
 def channel_chunks(proj: torch.Tensor, t: ChannelTerms, z: torch.Tensor, conv_state, state: torch.Tensor, cu_seqlens, slots, chunks: int,
-                   workspace, o: torch.Tensor) -> None:
-    """`channel_rows` and `channel_scan` of a step with many rows, by chunks of `channel_chunk()` rows on the matrix cores: proj
-    as there; z float32 [n, H*dk] = the second step of the decays' projection without its bias; `chunks`: the sequences' new rows
-    in chunks, every sequence's rounded up, added up; `workspace` gives the scratch; o float32 [n, H*dv].  The gate is not made."""
+                   workspace, gate: torch.Tensor, eps: float, out: torch.Tensor, weight=None, silu: bool = True, factor: float = 1.0) -> None:
+    """`channel_rows`, `channel_scan` and `heads_norm_gate` of a step with many rows, by chunks of `channel_chunk()` rows on the
+    matrix cores: proj as there; z float32 [n, H*dk] = the second step of the decays' projection without its bias; gate float32
+    [n, H*dv] (rows may be strided); `chunks`: the sequences' new rows in chunks, every sequence's rounded up, added up;
+    `workspace` gives the scratch; out bfloat16 [n, H*dv] (rows may be strided)."""
     n, width = proj.shape
     B = slots.shape[0]
     _req_columns(proj, (n, width), "channel_chunks.proj")
@@ -1555,19 +1556,24 @@ def channel_chunks(proj: torch.Tensor, t: ChannelTerms, z: torch.Tensor, conv_st
         _req_state(conv_state, (t.taps - 1) * t.channels, "channel_chunks")
     _req(cu_seqlens, "channel_chunks.cu_seqlens", torch.int32, (B + 1,))
     _req(slots, "channel_chunks.slots", torch.int32)
-    _req(o, "channel_chunks.o", torch.float32, (n, t.H * t.dv))
+    _req_columns(gate, (n, t.H * t.dv), "channel_chunks.gate")
+    _req_columns(out, (n, t.H * t.dv), "channel_chunks.out", torch.bfloat16)
+    if weight is not None:
+        _req(weight, "channel_chunks.weight", torch.float32, (t.dv,))
     if width < t.channels or not channel_chunks_serve(torch.bfloat16, t.dk, t.dv):
         raise KernelError(f"channel_chunks: heads of {t.dk} and {t.dv} in rows of {width} are not served")
     delta = t.b_off is not None
     rec = workspace.get("chunk_rec", (chunks * t.H * int(lib().tl_channel_record(t.dk, int(delta))),), torch.bfloat16)
     gam = workspace.get("chunk_gam", (chunks * t.H * int(lib().tl_channel_padded(t.dk)),), torch.float32)
     uf = workspace.get("chunk_u", (chunks * t.H * -(-t.dv // 16) * 1024,), torch.float32)
+    su = workspace.get("chunk_su", (chunks * t.H * -(-t.dv // 16) * int(lib().tl_channel_carried(t.dk)),), torch.bfloat16)
     _check(lib().tl_channel_chunks(_p(proj), proj.stride(0), t.G, t.H, t.dk, t.dv, int(t.b_off) if delta else -1, t.taps, _p(t.conv),
                                    _p(t.bias), _p(t.rate), ctypes.c_float(t.inv_tau), ctypes.c_float(t.qscale),
                                    ctypes.c_float(-1.0 if t.unit_eps is None else t.unit_eps), _p(z), _p(conv_state),
                                    ctypes.c_longlong(conv_state.stride(0) if t.taps else 0), _p(state),
                                    ctypes.c_longlong(state.stride(0)), _p(cu_seqlens), _p(slots), n, B, int(chunks), _p(rec), _p(gam),
-                                   _p(uf), _p(o), _stream()))
+                                   _p(uf), _p(su), _p(weight), _p(gate), gate.stride(0), int(bool(silu)), ctypes.c_float(eps),
+                                   ctypes.c_float(factor), _p(out), out.stride(0), _stream()))
     if t.taps:
         conv_carry(proj, 0, t.channels, t.taps, conv_state, cu_seqlens, slots)
 

@@ -183,11 +183,10 @@ class ChannelLinearMixer(ProjectedMixer):
             gate = proj[:, self.gate_off:self.gate_off + V] if not two_step else ws.get("clin_gate", (n, V), f32)
             if two_step:
                 self.gate_step(ctx, proj[:, t.g_off:t.g_off + t.g2.shape[1]], gate, "clin_inner")
-            o = ws.get("clin_o", (n, V), f32)
             C = ops.channel_chunk()
             chunks = int(sum(-(-int(r) // C) for r in ctx.host["n_new"]))
-            ops.channel_chunks(proj, t, z, conv_state, state, ctx.cu_seqlens, ctx.slots, chunks, ws, o)
-            ops.heads_norm_gate(o, gate, self.heads_n, self.eps, out, weight=self.norm_w, silu=not two_step, factor=self.factor)
+            ops.channel_chunks(proj, t, z, conv_state, state, ctx.cu_seqlens, ctx.slots, chunks, ws, gate, self.eps, out,
+                               weight=self.norm_w, silu=not two_step, factor=self.factor)
             return
         q, k, v = ws.get("clin_q", (n, Q), f32), ws.get("clin_k", (n, Q), f32), ws.get("clin_v", (n, V), f32)
         decay = ws.get("clin_decay", (n, K), f32)
