@@ -59,6 +59,56 @@ __device__ __forceinline__ float second_step(const T* __restrict__ w2, size_t ro
   return s0 + s1;
 }
 
+// z[c] = sum_r W2[first + c, r] * a[r] for c = lane, lane + 64, .. < count, handed to use(c, z).  LP lanes share a row's `rank`
+// numbers (16-byte pieces of at most LP * 8 bfloat16), so that a wave's load takes whole lines; all LP loads go before the sums
+template <int LP, typename F>
+__device__ __forceinline__ void shared_steps(const bf16* __restrict__ w2, size_t first, int count, const float* __restrict__ a, int rank,
+                                             int lane, F&& use) {
+  constexpr int PER = WAVE / LP;
+  const int j = lane % LP, at = lane / LP;                         // this lane's piece of rows at, at + PER, ..
+  const bool in = j * 8 < rank;
+  float x[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) x[e] = in ? a[j * 8 + e] : 0.f;
+  for (int c0 = 0; c0 < count; c0 += WAVE) {
+    bf16x8 v[LP];
+#pragma unroll
+    for (int p = 0; p < LP; ++p)
+      v[p] = *reinterpret_cast<const bf16x8*>(w2 + (first + min(c0 + p * PER + at, count - 1)) * rank + (in ? j * 8 : 0));
+    float mine = 0.f;
+#pragma unroll
+    for (int p = 0; p < LP; ++p) {
+      float s = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s = fmaf((float)v[p][e], x[e], s);
+      if constexpr (LP == 16) {
+        s = row16_sum(s);
+      } else {
+#pragma unroll
+        for (int o = 1; o < LP; o *= 2) s += __shfl_xor(s, o, WAVE);
+      }
+      // row c0 + lane lies in pass lane / PER, with the lanes that share place lane % PER
+      const float got = LP == 1 ? s : __shfl(s, (lane % PER) * LP, WAVE);
+      if (lane / PER == p) mine = got;
+    }
+    if (c0 + lane < count) use(c0 + lane, mine);
+  }
+}
+template <typename T, typename F>
+__device__ __forceinline__ void second_steps(const T* __restrict__ w2, size_t first, int count, const float* __restrict__ a, int rank, int lane,
+                                             F&& use) {
+  if constexpr (sizeof(T) == 2) {
+    if (rank % 8 == 0 && rank <= 128) {
+      if (rank <= 16) shared_steps<2>(w2, first, count, a, rank, lane, use);
+      else if (rank <= 32) shared_steps<4>(w2, first, count, a, rank, lane, use);
+      else if (rank <= 64) shared_steps<8>(w2, first, count, a, rank, lane, use);
+      else shared_steps<16>(w2, first, count, a, rank, lane, use);
+      return;
+    }
+  }
+  for (int c = lane; c < count; c += WAVE) use(c, second_step(w2, first + c, a, rank));
+}
+
 // One wave a unit of a row: a head of q, of k (G each), of v, of the decays (H each), of the gate (H, if made here), and
 // one unit for the betas.  `single`: every sequence brings one row, and the convolution's block is shifted on the way.
 template <typename T>
@@ -82,14 +132,21 @@ channel_rows_kernel(const float* __restrict__ proj, int width, ChannelTerms t, c
     auto value = [&](int c) {
       if (!t.taps) return row[c];
       const float* w = t.conv_w + (size_t)c * t.taps;
-      float acc = 0.f;
-      for (int j = 0; j < t.taps; ++j) {
-        const int back = t.taps - 1 - j, src = i - back;
-        const float u = src >= 0 ? row[c - (ptrdiff_t)back * width] : st[(size_t)(t.taps - 1 + src) * C + c];
-        acc = fmaf(w[j], u, acc);
-        if (single && back > 0 && j > 0) st[(size_t)(j - 1) * C + c] = u;
+      float u[CL_MAX_TAPS], wv[CL_MAX_TAPS];           // (all asked for before the block is shifted)
+#pragma unroll
+      for (int j = 0; j < CL_MAX_TAPS; ++j) {
+        if (j >= t.taps) break;
+        const int src = i - (t.taps - 1 - j);
+        u[j] = src >= 0 ? row[c - (ptrdiff_t)(t.taps - 1 - j) * width] : st[(size_t)(t.taps - 1 + src) * C + c];
+        wv[j] = w[j];
       }
-      if (single && t.taps > 1) st[(size_t)(t.taps - 2) * C + c] = row[c];
+      float acc = 0.f;
+#pragma unroll
+      for (int j = 0; j < CL_MAX_TAPS; ++j) {
+        if (j >= t.taps) break;
+        acc = fmaf(wv[j], u[j], acc);
+        if (single && j > 0) st[(size_t)(j - 1) * C + c] = u[j];
+      }
       return cl_silu(acc);
     };
     float x[CL_MAX_D / WAVE];
@@ -116,18 +173,17 @@ channel_rows_kernel(const float* __restrict__ proj, int width, ChannelTerms t, c
   unit -= 2 * t.G + t.H;
   if (unit < t.H) {                                // a head's decays
     const float rate = t.rate ? -expf(t.rate[unit]) : 0.f;
-    for (int c = lane; c < t.dk; c += WAVE) {
+    second_steps(a2, (size_t)unit * t.dk, t.dk, row + t.a_off, t.a_rank, lane, [&](int c, float z) {
       const int at = unit * t.dk + c;
-      const float z = second_step(a2, at, row + t.a_off, t.a_rank) + (t.bias ? t.bias[at] : 0.f);
-      decay[(size_t)n * t.H * t.dk + at] = expf(cl_log_decay(z, t.rate != nullptr, rate, t.inv_tau));
-    }
+      decay[(size_t)n * t.H * t.dk + at] = expf(cl_log_decay(z + (t.bias ? t.bias[at] : 0.f), t.rate != nullptr, rate, t.inv_tau));
+    });
     return;
   }
   unit -= t.H;
   if (t.g_rank) {
     if (unit < t.H) {                              // a head's gates
-      for (int c = lane; c < t.dv; c += WAVE)
-        gate[(size_t)n * V + unit * t.dv + c] = second_step(g2, unit * t.dv + c, row + t.g_off, t.g_rank);
+      second_steps(g2, (size_t)unit * t.dv, t.dv, row + t.g_off, t.g_rank, lane,
+                   [&](int c, float z) { gate[(size_t)n * V + unit * t.dv + c] = z; });
       return;
     }
     unit -= t.H;
@@ -171,6 +227,17 @@ channel_scan_kernel(const float* __restrict__ q, const float* __restrict__ k, co
   if (n_new == 0) return;
   const int kh = h / (H / G);
   float* S_g = state + (long long)slots[b] * stride + ((size_t)h * dv + c0 + cg * DC) * dk;
+  // a single token's gate (and the norm's weight), asked for before anything waits
+  constexpr int GC = 2;                                          // columns of a head a thread, at most
+  float gt[GC], wt[GC];
+  if (!z.o) {
+#pragma unroll
+    for (int r = 0; r < GC; ++r) {
+      const int c = threadIdx.x + r * blockDim.x;
+      gt[r] = c < dv ? z.gate[(size_t)row0 * z.gate_stride + (size_t)h * dv + c] : 0.f;
+      wt[r] = c < dv && z.w ? z.w[c] : 1.f;
+    }
+  }
   float S[DC][R * VEC];
 #pragma unroll
   for (int c = 0; c < DC; ++c)
@@ -278,9 +345,11 @@ channel_scan_kernel(const float* __restrict__ q, const float* __restrict__ k, co
   float sum = 0.f;
   for (int w = 0; w < NT / WAVE; ++w) sum += sh[w];
   const float f = z.factor / sqrtf(sum / (float)dv + z.eps);
-  for (int c = t; c < dv; c += NT) {
-    const float g = z.gate[(size_t)row0 * z.gate_stride + (size_t)h * dv + c];
-    const float a = os[c] * f * (z.w ? z.w[c] : 1.f) * (z.gate_silu ? cl_silu(g) : cl_sigmoid(g));
+#pragma unroll
+  for (int r = 0; r < GC; ++r) {
+    const int c = t + r * NT;
+    if (c >= dv) break;
+    const float a = os[c] * f * wt[r] * (z.gate_silu ? cl_silu(gt[r]) : cl_sigmoid(gt[r]));
     const size_t at = (size_t)row0 * z.out_stride + (size_t)h * dv + c;
     if (z.out_f32) ((float*)z.out)[at] = a;
     else ((bf16*)z.out)[at] = (bf16)a;
@@ -361,8 +430,8 @@ int tl_channel_scan(const float* q, const float* k, const float* v, const float*
   // parts, so that every compute unit has work
   int DC = 1, threads = 256;
   if (!o) {
-    while (DC < 8 && (256 / 16) * DC < dv) DC *= 2;
-    while ((threads / 16) * DC < dv) threads *= 2;             // (dv up to 256: 512 threads)
+    if (dv > 64) threads = 512;
+    while ((threads / 16) * DC < dv) DC *= 2;                  // (dv up to 256: 8 columns)
   } else {
     const long long units = (long long)H * B;
     while (DC < 4 && (256 / 16) * DC < dv && units * ((dv + 32 * DC - 1) / (32 * DC)) >= 512) DC *= 2;

@@ -27,8 +27,8 @@ __global__ void embed_kernel(const T* __restrict__ table, const int* __restrict_
 
 // The same with a second table read by pairs of tokens, and a norm of the sum: row (previous * mul_prev + current * mul_cur)
 // mod buckets of `pairs`, row `buckets` for a sequence's first token.  The previous token of a sequence's first row of the
-// step lies in `last`; the workgroup of that row alone reads and then replaces it.  One workgroup a row; the row's sum goes
-// through `out` (every thread reads back what it wrote).
+// step lies in `last`; the workgroup of that row alone reads and then replaces it.  One workgroup a row, which stays in
+// registers (IT > 0: H % 4 == 0, H <= 1024 * IT) or goes through `out` (every thread reads back what it wrote).
 struct PairTerms {
   const int* row_pos;
   const int* row_seq;
@@ -37,7 +37,12 @@ struct PairTerms {
   int* last;
   long long buckets, mul_prev, mul_cur;
 };
-template <typename T>
+__device__ __forceinline__ f32x4 row4(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+__device__ __forceinline__ f32x4 row4(const bf16* p) {
+  const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+  return f32x4{(float)v[0], (float)v[1], (float)v[2], (float)v[3]};
+}
+template <typename T, int IT>
 __global__ void __launch_bounds__(256)
 embed_pairs_kernel(const T* __restrict__ table, const int* __restrict__ ids, int H, float scale, const T* __restrict__ pairs, PairTerms k,
                    const float* __restrict__ w, float eps, float* __restrict__ out) {
@@ -45,14 +50,29 @@ embed_pairs_kernel(const T* __restrict__ table, const int* __restrict__ ids, int
   __shared__ int s_prev;
   const int n = blockIdx.x;
   const T* row = table + (size_t)ids[n] * H;
+  constexpr int R = IT > 0 ? IT : 1;
+  f32x4 v[R], wv[R];                                   // (asked for before the previous token is known)
+  if constexpr (IT > 0) {
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int i = (threadIdx.x + 256 * r) * 4;
+      if (i < H) {
+        v[r] = row4(row + i);
+        if (w) wv[r] = *reinterpret_cast<const f32x4*>(w + i);
+      }
+    }
+  }
   const T* second = nullptr;
   if (pairs) {
-    const int b = k.row_seq[n], row0 = k.cu_seqlens[b];
     if (threadIdx.x == 0) {
-      int prev = n > row0 ? ids[n - 1] : k.last[k.slots[b]];
-      if (k.row_pos[n] == 0) prev = -1;
-      s_prev = prev;
-      if (n == row0) k.last[k.slots[b]] = ids[k.cu_seqlens[b + 1] - 1];
+      const int b = k.row_seq[n], before = n > 0 ? ids[n - 1] : -1, pos = k.row_pos[n];
+      const int row0 = k.cu_seqlens[b], end = k.cu_seqlens[b + 1], slot = k.slots[b];
+      int prev = before;
+      if (n == row0) {
+        prev = k.last[slot];
+        k.last[slot] = ids[end - 1];
+      }
+      s_prev = pos == 0 ? -1 : prev;
     }
     __syncthreads();
     const int prev = s_prev;
@@ -62,6 +82,28 @@ embed_pairs_kernel(const T* __restrict__ table, const int* __restrict__ ids, int
   }
   float* o = out + (size_t)n * H;
   float ss = 0.f;
+  if constexpr (IT > 0) {
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int i = (threadIdx.x + 256 * r) * 4;
+      if (i >= H) continue;
+      v[r] *= scale;
+      if (second) v[r] += row4(second + i);
+      ss += v[r][0] * v[r][0] + v[r][1] * v[r][1] + v[r][2] * v[r][2] + v[r][3] * v[r][3];
+    }
+    if (w) ss = block_sum<256>(ss, sh);
+    const float root = sqrtf(ss / (float)H + eps);
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const int i = (threadIdx.x + 256 * r) * 4;
+      if (i >= H) continue;
+      if (w)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[r][e] = (v[r][e] / root) * wv[r][e];
+      *reinterpret_cast<f32x4*>(o + i) = v[r];
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < H; i += 256) {
     float a = to_f32(row[i]) * scale;
     if (second) a += to_f32(second[i]);
@@ -797,10 +839,20 @@ int tl_embed_pairs(const void* table, int table_dt, const int* ids, int n, int H
   TL_REQUIRE(table_dt == DT_F32 || table_dt == DT_BF16, "embed_pairs: unknown dtype code %d", table_dt);
   if (n == 0) return 0;
   const PairTerms k{row_pos, row_seq, cu_seqlens, slots, last, buckets, mul_prev, mul_cur};
-  if (table_dt == DT_F32)
-    embed_pairs_kernel<float><<<n, 256, 0, st>>>((const float*)table, ids, H, scale, (const float*)pairs, k, w, eps, out);
-  else
-    embed_pairs_kernel<bf16><<<n, 256, 0, st>>>((const bf16*)table, ids, H, scale, (const bf16*)pairs, k, w, eps, out);
+  const bool vec = H % 4 == 0 && H <= 8192 && ((uintptr_t)table | (uintptr_t)pairs | (uintptr_t)w | (uintptr_t)out) % 16 == 0;
+#define TL_EP(IT)                                                                                                               \
+  do {                                                                                                                          \
+    if (table_dt == DT_F32)                                                                                                     \
+      embed_pairs_kernel<float, IT><<<n, 256, 0, st>>>((const float*)table, ids, H, scale, (const float*)pairs, k, w, eps, out); \
+    else                                                                                                                        \
+      embed_pairs_kernel<bf16, IT><<<n, 256, 0, st>>>((const bf16*)table, ids, H, scale, (const bf16*)pairs, k, w, eps, out);   \
+  } while (0)
+  if (!vec) TL_EP(0);
+  else if (H <= 1024) TL_EP(1);
+  else if (H <= 2048) TL_EP(2);
+  else if (H <= 4096) TL_EP(4);
+  else TL_EP(8);
+#undef TL_EP
   TL_LAUNCH_CHECK("embed_pairs");
   return 0;
 }
