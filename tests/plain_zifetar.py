@@ -96,12 +96,15 @@ def unit(t):
     return t / torch.sqrt((t * t).sum(dim=-1, keepdim=True) + 1e-6)
 
 
-def linear_heads(q, k, v, g, beta=None, S=None):
+def linear_heads(q, k, v, g, beta=None, S=None, left=None):
     """q, k, g [T, H, d], v [T, H, dv]: S <- g S + k u^T, o = S^T q, row by row; u = v, or with `beta`
-    [T, H] the delta rule's beta (v - (g S)^T k)."""
+    [T, H] the delta rule's beta (v - (g S)^T k).  `left`: a list that receives, per row, what is left of o when its
+    terms have cancelled (its length over the length of the sum of their magnitudes, times sqrt(d): about 1 for terms of
+    any sign; the smallest of the heads): a norm over the head makes what is left large again, with the rounding of the
+    terms."""
     T, H, d = q.shape
     S = torch.zeros(H, d, v.shape[-1], dtype=q.dtype) if S is None else S
-    out = []
+    out, kept = [], []
     for t in range(T):
         S = g[t][:, :, None] * S
         u = v[t]
@@ -109,6 +112,9 @@ def linear_heads(q, k, v, g, beta=None, S=None):
             u = beta[t][:, None] * (u - (S * k[t][:, :, None]).sum(dim=1))
         S = S + k[t][:, :, None] * u[:, None, :]
         out.append((S * q[t][:, :, None]).sum(dim=1))
+        kept.append(d ** 0.5 * (out[-1].norm(dim=-1) / (S * q[t][:, :, None]).abs().sum(dim=1).norm(dim=-1).clamp(min=1e-30)).min())
+    if left is not None:
+        left.append(torch.stack(kept))
     return torch.stack(out), S
 
 
@@ -123,30 +129,30 @@ def delta_inputs(h, w, p, m):
     return q, k, v.view(T, H, dv), g, torch.sigmoid(h @ w[p + "b"].T)
 
 
-def channel_delta(h, w, p, m, pos, eps):
+def channel_delta(h, w, p, m, pos, eps, left=None):
     T, H, dv = h.shape[0], m["heads"], m["vdim"]
-    o, _ = linear_heads(*delta_inputs(h, w, p, m))
+    o, _ = linear_heads(*delta_inputs(h, w, p, m), left=left)
     gate = torch.sigmoid((h @ w[p + "g1"].T) @ w[p + "g2"].T)
     return ((rms(o, eps) * w[p + "norm"]).reshape(T, H * dv) * gate) @ w[p + "o"].T
 
 
-def retention(h, w, p, m, pos, eps):
+def retention(h, w, p, m, pos, eps, left=None):
     T, H, d, dv = h.shape[0], m["heads"], m["dim"], m["vdim"]
     q = rotate((h @ w[p + "q"].T).view(T, H, d), pos, m.get("rot"))
     k = rotate((h @ w[p + "k"].T).view(T, H, d), pos, m.get("rot")) * d ** -0.5
     v = (h @ w[p + "v"].T).view(T, H, dv)
     g = torch.tensor(m["decay"], dtype=h.dtype)[None, :, None].expand(T, H, d)
-    o, _ = linear_heads(q, k, v, g)
+    o, _ = linear_heads(q, k, v, g, left=left)
     return (rms(o, eps).reshape(T, H * dv) * silu(h @ w[p + "g"].T)) @ w[p + "o"].T
 
 
-def gated_linear(h, w, p, m, eps):
+def gated_linear(h, w, p, m, eps, left=None):
     T, H, d, dv = h.shape[0], m["heads"], m["dim"], m["vdim"]
     q = (h @ w[p + "q"].T).view(T, H, d) * d ** -0.5
     k = (h @ w[p + "k"].T).view(T, H, d)
     v = (h @ w[p + "v"].T).view(T, H, dv)
     z = (h @ w[p + "a1"].T) @ w[p + "a2"].T + w[p + "a2.b"]
-    o, _ = linear_heads(q, k, v, torch.sigmoid(z).pow(1.0 / m["tau"]).view(T, H, d))
+    o, _ = linear_heads(q, k, v, torch.sigmoid(z).pow(1.0 / m["tau"]).view(T, H, d), left=left)
     return ((rms(o, eps) * w[p + "norm"]).reshape(T, H * dv) * silu(h @ w[p + "g"].T)) @ w[p + "o"].T
 
 
@@ -171,9 +177,9 @@ def chunked_attention(h, w, p, m, pos, eps):
     return o.transpose(0, 1).reshape(T, H * dv) @ w[p + "o"].T
 
 
-def parallel(h, w, p, m, pos, eps):
+def parallel(h, w, p, m, pos, eps, left=None):
     return (m["left_scale"] * chunked_attention(h, w, p + "left.", m["left"], pos, eps)
-            + m["right_scale"] * gated_linear(h, w, p + "right.", m["right"], eps))
+            + m["right_scale"] * gated_linear(h, w, p + "right.", m["right"], eps, left))
 
 
 MIXERS = {"channel_delta": channel_delta, "retention": retention, "parallel": parallel}
@@ -209,16 +215,16 @@ def routed_ff(h, w, p, mlp, margins=None):
 
 # ---- the model --------------------------------------------------------------------------------------
 
-def forward(w, cfg, ids, dtype=F64, streams=None, margins=None):
+def forward(w, cfg, ids, dtype=F64, streams=None, margins=None, left=None):
     """Logits [T, vocab] of one sequence.  `streams`: a list that receives the stream after every
-    layer; `margins`: see `route`."""
+    layer; `margins`: see `route`; `left`: see `linear_heads`."""
     w = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in w.items()}
     eps = cfg["norm"]["eps"]
     pos = torch.arange(len(ids))
     x = embedding(w, cfg, ids)
     for i, layer in enumerate(cfg["layers"]):
         p = f"l{i}."
-        y = MIXERS[layer["type"]](norm(x, eps, w[p + "norm1"]), w, p + "mix.", layer["mixer"], pos, eps)
+        y = MIXERS[layer["type"]](norm(x, eps, w[p + "norm1"]), w, p + "mix.", layer["mixer"], pos, eps, left)
         x = x + norm(y, eps, w[p + "norm1b"])
         if layer.get("mlp"):
             y = routed_ff(norm(x, eps, w[p + "norm2"]), w, p + "mlp.", layer["mlp"], margins)

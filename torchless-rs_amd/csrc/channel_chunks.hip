@@ -861,7 +861,7 @@ int tl_channel_chunks(const float* proj, int width, int G, int H, int dk, int dv
              CC_MAX_DK, CL_MAX_D);
   const int C = 2 * G * dk + H * dv;
   TL_REQUIRE(C <= width && b_off + (b_off < 0 ? 0 : H) <= width, "channel_chunks: a row of %d is too short", width);
-  TL_REQUIRE(taps >= 0 && taps <= CL_MAX_TAPS && (taps == 0 || (conv_w && conv_state && conv_stride >= (long long)(taps - 1) * C)),
+  TL_REQUIRE(taps >= 0 && taps <= CL_MAX_TAPS && (taps == 0 || (conv_w && (conv_state || taps == 1) && conv_stride >= (long long)(taps - 1) * C)),
              "channel_chunks: a convolution of %d taps without weights, or a block too small", taps);
   TL_REQUIRE(proj && z && state && cu && slots && rec && gam && uf && su && gate && out, "channel_chunks: a buffer is missing");
   TL_REQUIRE(((uintptr_t)rec | (uintptr_t)gam | (uintptr_t)uf | (uintptr_t)su) % 16 == 0, "channel_chunks: a buffer off 16 bytes");

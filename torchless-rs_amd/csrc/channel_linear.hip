@@ -386,7 +386,7 @@ int tl_channel_rows(const float* proj, int width, int G, int H, int dk, int dv, 
   TL_REQUIRE(C <= width && a_rank > 0 && a_off >= 0 && a_off + a_rank <= width && g_rank >= 0 && (g_rank == 0 || (g_off >= 0 && g_off + g_rank <= width)),
              "channel_rows: a row of %d does not hold the inner rows of %d and %d", width, a_rank, g_rank);
   TL_REQUIRE(taps >= 0 && taps <= CL_MAX_TAPS, "channel_rows: %d taps (up to %d)", taps, CL_MAX_TAPS);
-  TL_REQUIRE(taps == 0 || (conv_w && conv_state && row_seq && cu_seqlens && slots && stride >= (long long)(taps - 1) * C),
+  TL_REQUIRE(taps == 0 || (conv_w && (conv_state || taps == 1) && row_seq && cu_seqlens && slots && stride >= (long long)(taps - 1) * C),
              "channel_rows: a convolution without weights, or a block too small for %d rows of %d", taps - 1, C);
   TL_REQUIRE(proj && a2 && q && k && v && decay && (b_off < 0 || beta) && (g_rank == 0 || (g2 && gate)), "channel_rows: a buffer is missing");
   TL_REQUIRE(!single || n == B, "channel_rows: %d rows of %d sequences are not one row each", n, B);

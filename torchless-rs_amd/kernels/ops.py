@@ -1484,7 +1484,7 @@ def channel_rows(proj: torch.Tensor, t: ChannelTerms, conv_state, row_seq, cu_se
                                  _p(conv_state), ctypes.c_longlong(conv_state.stride(0) if t.taps else 0), _p(row_seq),
                                  _p(cu_seqlens), _p(slots), n, B, int(bool(single)), _p(q), _p(k), _p(v), _p(decay), _p(beta),
                                  _p(gate), _stream()))
-    if t.taps and not single:
+    if t.taps > 1 and not single:
         conv_carry(proj, 0, t.channels, t.taps, conv_state, cu_seqlens, slots)
 
 
@@ -1574,7 +1574,7 @@ def channel_chunks(proj: torch.Tensor, t: ChannelTerms, z: torch.Tensor, conv_st
                                    ctypes.c_longlong(state.stride(0)), _p(cu_seqlens), _p(slots), n, B, int(chunks), _p(rec), _p(gam),
                                    _p(uf), _p(su), _p(weight), _p(gate), gate.stride(0), int(bool(silu)), ctypes.c_float(eps),
                                    ctypes.c_float(factor), _p(out), out.stride(0), _stream()))
-    if t.taps:
+    if t.taps > 1:
         conv_carry(proj, 0, t.channels, t.taps, conv_state, cu_seqlens, slots)
 
 
